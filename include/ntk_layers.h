@@ -70,6 +70,11 @@ int ntk_residual_add(float* x, const float* a, const float* b, int n, void* stre
 
 /* out[t][:] = table[tokens[t]][:] * scale */
 int ntk_embed_dense_scaled(float* out, const void* table, int tdtype, const int* tokens, int T, int vocab, int width, float scale, void* stream);
+/* ... and a row of a second table picked by the token and the one before it: out[t][:] = table[tokens[t]][:] * scale + bigram[r][:] with
+ * r = (tokens[t-1] * mul_prev + tokens[t] * mul_cur) mod buckets (64-bit), and r = buckets for a sequence's first token (pos0 + t == 0); bigram [buckets + 1][width]
+ * in the table's dtype.  prev is the token before tokens[0] (unused when pos0 == 0). */
+int ntk_embed_bigram(float* out, const void* table, const void* bigram, int tdtype, const int* tokens, int prev, int pos0, int T, int vocab, int width, float scale,
+                     int buckets, long long mul_prev, long long mul_cur, void* stream);
 /* x[i] *= s */
 int ntk_scale(float* x, long long n, float s, void* stream);
 /* Layer norm with weight and bias: y[t][:] (+)= (x[t] - mean) / sqrt(var + eps) * w + b, var = mean of the squared deviations (two passes).
@@ -206,6 +211,10 @@ typedef struct ntk_window_prepare_desc {
     const float* v_other; int ld_other; float v_blend;
     float* v_keep; int ld_keep;
     int pos0, T;
+    /* q_norm [H*maps*dn] / k_norm [G*maps*dn] device F32 (each may be NULL): the token's whole q (after bias and temperature) / whole k (after bias) divided by
+     * sqrt(mean(x^2) + norm_eps), the mean over ALL heads at once, times the weight, ahead of the rotation.
+     * k == NULL (then v, cache and everything of theirs too): only q is treated -- a layer that reads the cache rows of another one. */
+    const float* q_norm; const float* k_norm; float norm_eps;
 } ntk_window_prepare_desc;
 int ntk_window_prepare_ex(const ntk_window_prepare_desc* d, void* stream);
 /* a_m = softmax_j(scale * q_m . k_m[j]) V over the visible j (j <= p, and p - j < window if window > 0), per map m.
@@ -230,8 +239,12 @@ typedef struct ntk_window_attention_desc {
      * sink != 0: one more term exp(0) in the softmax's denominator (a key of score 0 that carries no value): p_j = exp(s_j) / (1 + sum exp(s)). */
     int mask_mode; float softcap; int sink;
     /* gate != NULL: the result (after the pair, the unit norm and out_scale) times sigmoid(gate[t][h][c]), gate rows ldg floats apart: an elementwise output gate
-     * inside the launch that writes the result */
+     * inside the launch that writes the result; head_gate != 0: one number per token and head, gate[t][h] */
     const float* gate; int ldg;
+    /* keep_first > 0 (NTK_MASK_SLIDING): positions j < keep_first stay visible to every later query beside the window; their keys are the cache rows as they are.
+     * sinks != NULL (device F32 [H]): the sink's score is sinks[h] (unscaled, once per head) instead of 0; `sink` need not be set. */
+    int head_gate, keep_first;
+    const float* sinks;
 } ntk_window_attention_desc;
 #define NTK_MASK_SLIDING 0
 #define NTK_MASK_CHUNKS 1
@@ -323,6 +336,8 @@ int ntk_glu(float* a, const float* gu, int rows, int ff, float limit, float alph
 /* ... with a cubic term inside the sigmoid, g' * sigmoid(alpha * (g' + cubic * g'^3)) * (u' + up_offset) (the tanh form of gelu: see ntk_dense_desc), and gu rows
  * ldgu floats apart (gate values at [0, ff), up values at [ff, 2 ff)) */
 int ntk_glu_cubic(float* a, const float* gu, int ldgu, int rows, int ff, float limit, float alpha, float cubic, float up_offset, void* stream);
+/* the general form with the output rows lda floats apart (lda >= ff) */
+int ntk_glu_rows(float* a, int lda, const float* gu, int ldgu, int rows, int ff, float limit, float alpha, float cubic, float up_offset, void* stream);
 /* out[t][:] = sum_s wts[t][s] * d[where[t*top+s]][:] + (sgate ? sgate[t] : 1) * shared[t][:] (if shared): the experts' sum on its own, for layers that norm it before
  * it joins the stream */
 int ntk_moe_sum(float* out, const float* d, const int* where, const float* wts, const float* shared, const float* sgate, int T, int top, int n, void* stream);

@@ -13,6 +13,8 @@ namespace nt {
         if (st__ != NTK_OK) return st__;      \
     } while (0)
 
+// inputs up to which a layer's two output products are one (the few-row form keeps the whole row of inputs in LDS: 64 KB)
+static constexpr int kJoinedInputs = 16384;
 static constexpr float kGluAlpha = 1.702f;   // the slope of the clipped gated unit's activation
 static StackForm parallel_form() { return StackForm{}; }
 static StackForm sequential_form() {
@@ -31,11 +33,18 @@ static StackForm scaled_form() {
     f.mask_chunks = true; f.attention_sink = true; f.attention_gate = true; f.rot_halves = true; f.latent_head_gate = true;
     return f;
 }
+static StackForm dense_parallel_form() {
+    StackForm f;
+    f.dense_parallel = true; f.loop_projection = false; f.clipped_glu = false;
+    f.rot_halves = true; f.blended_rotation = true; f.learned_sinks = true; f.attention_gate = true; f.attention_head_gate = true; f.whole_qk_norm = true;
+    return f;
+}
 // what the gated form's mechanisms fix
 static constexpr float kGeluAlpha = 1.5957691216057308f;   // 2 sqrt(2 / pi): 0.5 (1 + tanh y) = sigmoid(2 y)
 static constexpr float kGeluCubic = 0.044715f;
 static constexpr float kDeltaDecayRate = 0.6065306597126334f;   // exp(-1/2): w = exp(-rate * sigmoid(.))
 static constexpr float kUnitKeyEps = 1e-6f;
+static FamilyRegistrar reg_zalazen("Zalazen", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(dense_parallel_form())); });
 static FamilyRegistrar reg_fifotar("Fifotar", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(scaled_form())); });
 static FamilyRegistrar reg_tubazen("Tubazen", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(gated_form())); });
 static FamilyRegistrar reg_fabolorn("Fabolorn", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(parallel_form())); });
@@ -63,6 +72,27 @@ static bool need_int(const Json& o, const char* key, int& out, std::string& err,
     return true;
 }
 
+// rotary frequencies base^(-2i/dims), optionally blended with themselves over `factor` along a ramp over the pair index; cos and sin then carry *mag
+static std::vector<double> blended_frequencies(const Json& rot, int dims, float* mag) {
+    const double base = rot.at("base").number(10000.0);
+    const int half = dims / 2;
+    std::vector<double> f((size_t)std::max(half, 1));
+    for (int i = 0; i < half; ++i) f[(size_t)i] = std::pow(base, -2.0 * i / dims);
+    *mag = 1.0f;
+    if (rot.has("scaling")) {
+        const Json& sc = rot.at("scaling");
+        const double factor = sc.at("factor").number(1.0), orig = sc.at("original").number(1.0), fast = sc.at("fast").number(1.0), slow = sc.at("slow").number(1.0);
+        auto where_dim = [&](double turns) { return dims * std::log(orig / (2.0 * M_PI * turns)) / (2.0 * std::log(base)); };
+        const double lo = std::max(std::floor(where_dim(fast)), 0.0), hi = std::min(std::ceil(where_dim(slow)), (double)dims - 1.0);
+        for (int i = 0; i < half; ++i) {
+            const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            f[(size_t)i] = f[(size_t)i] / factor * ramp + f[(size_t)i] * (1.0 - ramp);
+        }
+        *mag = (float)(0.1 * std::log(factor) + 1.0);
+    }
+    return f;
+}
+
 int LayerStackModel::parse_mixer(const Json& L, const std::string& type, LatentMixer& m) {
     const Json& mx = L.at("mixer");
     const std::string where = "mixer '" + type + "'";
@@ -87,22 +117,7 @@ int LayerStackModel::parse_mixer(const Json& L, const std::string& type, LatentM
     if (!rot.is_object() || !rot.at("base").is_number()) return fail(NTK_E_FORMAT, where + ": 'rot' is missing");
     m.rot_dims = rot.has("dims") ? (int)rot.at("dims").integer() : m.rot_dim;
     if (m.rot_dims < 0 || (m.rot_dims & 1) || m.rot_dims > m.rot_dim) return fail(NTK_E_FORMAT, where + ": rot.dims must be even and at most rot_dim");
-    const double base = rot.at("base").number();
-    const int half = m.rot_dims / 2;
-    std::vector<double> f((size_t)std::max(half, 1));
-    for (int i = 0; i < half; ++i) f[(size_t)i] = std::pow(base, -2.0 * i / m.rot_dims);
-    m.rot_mag = 1.0f;
-    if (rot.has("scaling")) {
-        const Json& sc = rot.at("scaling");
-        const double factor = sc.at("factor").number(1.0), orig = sc.at("original").number(1.0), fast = sc.at("fast").number(1.0), slow = sc.at("slow").number(1.0);
-        auto where_dim = [&](double turns) { return m.rot_dims * std::log(orig / (2.0 * M_PI * turns)) / (2.0 * std::log(base)); };
-        const double lo = std::max(std::floor(where_dim(fast)), 0.0), hi = std::min(std::ceil(where_dim(slow)), (double)m.rot_dims - 1.0);
-        for (int i = 0; i < half; ++i) {
-            const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
-            f[(size_t)i] = f[(size_t)i] / factor * ramp + f[(size_t)i] * (1.0 - ramp);
-        }
-        m.rot_mag = (float)(0.1 * std::log(factor) + 1.0);
-    }
+    const std::vector<double> f = blended_frequencies(rot, m.rot_dims, &m.rot_mag);
     m.rot_layout = form_.rot_halves ? NTK_ROT_HALVES : NTK_ROT_NEIGHBOURS;
     m.head_gate = form_.latent_head_gate;
     m.rot_freq = (double*)dev_alloc(f.size() * sizeof(double));
@@ -144,20 +159,30 @@ int LayerStackModel::parse_window(const Json& L, WindowMixer& m) {
     m.maps = mx.has("diff") ? 2 : 1;
     m.diff = (float)mx.at("diff").number(0.0);
     m.window = 0;
-    if (mx.has("mask") && !need_int(mx.at("mask"), "size", m.window, err_, where + " mask")) return NTK_E_FORMAT;
+    const bool masked = mx.has("mask") && !mx.at("mask").is_null();
+    if (masked && !need_int(mx.at("mask"), "size", m.window, err_, where + " mask")) return NTK_E_FORMAT;
+    if (form_.dense_parallel && masked) {
+        m.keep_first = (int)mx.at("mask").at("keep_first").integer(0);
+        if (m.keep_first < 0) return fail(NTK_E_FORMAT, where + ": mask.keep_first must not be negative");
+    }
     m.mask_mode = form_.mask_chunks ? NTK_MASK_CHUNKS : NTK_MASK_SLIDING;
     m.sink = form_.attention_sink;
     m.gated = form_.attention_gate;
+    m.head_gate = form_.attention_head_gate;
+    if (form_.dense_parallel && mx.at("kv_from").is_number()) {
+        m.kv_from = (int)mx.at("kv_from").integer();
+        if (m.kv_from < 0) return fail(NTK_E_FORMAT, where + ": kv_from must name a layer");
+    }
     m.softcap = (float)mx.at("softcap").number(0.0);
     if (m.softcap < 0.0f) return fail(NTK_E_FORMAT, where + ": 'softcap' must be positive");
     m.v_mix = form_.scaled && mx.at("v_mix").truth();
     m.rot_dims = 0;
     std::vector<double> f(1, 0.0);
-    if (mx.has("rot")) {
+    if (mx.has("rot") && !mx.at("rot").is_null()) {
         const Json& rot = mx.at("rot");
         m.rot_dims = rot.has("dims") ? (int)rot.at("dims").integer() : m.dim;
         if (m.rot_dims < 0 || (m.rot_dims & 1) || m.rot_dims > m.dim) return fail(NTK_E_FORMAT, where + ": rot.dims must be even and at most dim");
-        f = wavelength_scaled_frequencies(rot, m.rot_dims);
+        f = form_.blended_rotation ? blended_frequencies(rot, m.rot_dims, &m.rot_mag) : wavelength_scaled_frequencies(rot, m.rot_dims);
     }
     m.rot_freq = (double*)dev_alloc(f.size() * sizeof(double));
     if (!m.rot_freq) return fail(NTK_E_NOMEM, "out of device memory");
@@ -244,9 +269,11 @@ int LayerStackModel::parse_parallel(const Json& L, ParallelMixer& m) {
 
 int LayerStackModel::parse_mlp(const Json& ml, const std::string& where, StackLayer& S) {
     const std::string kind = ml.at("kind").is_string() ? ml.at("kind").str : "moe";
-    if (kind == "dense" && form_.scaled) {
-        S.mlp_kind = kMlpClipped;
+    if (kind == "dense" && (form_.scaled || form_.dense_parallel)) {
+        S.mlp_kind = kMlpUnit;
         if (!need_int(ml, "ff", S.cff.ff, err_, where)) return NTK_E_FORMAT;
+        S.cff.limit = INFINITY;
+        if (form_.dense_parallel) return NTK_OK;
         S.cff.limit = ml.at("limit").is_number() ? (float)ml.at("limit").number() : INFINITY;
         if (!(S.cff.limit > 0.0f)) return fail(NTK_E_FORMAT, where + ": 'limit' must be positive");
         return NTK_OK;
@@ -256,7 +283,7 @@ int LayerStackModel::parse_mlp(const Json& ml, const std::string& where, StackLa
         if (!need_int(ml, "ff", form_.gated ? S.gff.ff : S.ffn.ff, err_, where)) return NTK_E_FORMAT;
         return NTK_OK;
     }
-    if (form_.gated || form_.scaled) return fail(NTK_E_FORMAT, where + ": this family has the dense feed-forward only");
+    if (form_.gated || form_.scaled || form_.dense_parallel) return fail(NTK_E_FORMAT, where + ": this family has the dense feed-forward only");
     if (kind != "moe") return fail(NTK_E_FORMAT, where + ": unknown kind '" + kind + "'");
     S.mlp_kind = kMlpMoe;
     MoeFeedForward& M = S.mlp;
@@ -306,6 +333,18 @@ int LayerStackModel::parse(const ModelFolder& f) {
         if (logit_softcap_ < 0.0f) return fail(NTK_E_FORMAT, "config: logit_softcap must be positive");
         norm_offset_ = 0.0f;
     }
+    if (form_.dense_parallel) {
+        const Json& e = c.at("embedding");
+        embed_scale_ = (float)e.at("scale").number(1.0);
+        norm_offset_ = 0.0f;
+        if (e.at("bigram").is_object()) {
+            const Json& b = e.at("bigram");
+            if (!need_int(b, "buckets", buckets_, err_, "config: embedding.bigram")) return NTK_E_FORMAT;
+            if (!b.at("mul_prev").is_number() || !b.at("mul_cur").is_number()) return fail(NTK_E_FORMAT, "config: embedding.bigram needs mul_prev and mul_cur");
+            mul_prev_ = b.at("mul_prev").integer();
+            mul_cur_ = b.at("mul_cur").integer();
+        }
+    }
     if (c.at("bos").is_number()) info_.bos = (int)c.at("bos").integer();
     if (c.at("eos").is_number()) info_.eos = (int)c.at("eos").integer();
     const Json& ls = c.at("layers");
@@ -316,7 +355,9 @@ int LayerStackModel::parse(const ModelFolder& f) {
         StackLayer& S = layers_[i];
         S.type = L.at("type").str;
         // which mixers a form lists: the parallel form's layers read two norms of one input, so its mixers are the latent kinds it was built around
-        if (form_.scaled && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
+        if (form_.dense_parallel && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
+        else if (form_.dense_parallel) return fail(NTK_E_FORMAT, "layer " + std::to_string(i) + ": unknown mixer type '" + S.type + "'");
+        else if (form_.scaled && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
         else if (form_.scaled && S.type == "latent_attention") { S.mixer = kMixLatent; LS_TRY(parse_mixer(L, S.type, S.mix)); }
         else if (form_.scaled && S.type == "delta") { S.mixer = kMixGatedDelta; LS_TRY(parse_gated_delta(L, S.gdl)); has_state_ = true; }
         else if (form_.scaled) return fail(NTK_E_FORMAT, "layer " + std::to_string(i) + ": unknown mixer type '" + S.type + "'");
@@ -334,7 +375,16 @@ int LayerStackModel::parse(const ModelFolder& f) {
     // the order of layer runs
     const int n = (int)layers_.size();
     runs_.clear();
-    has_loop_ = c.has("loop") && !form_.gated && !form_.scaled;   // (the gated form's depth weights are per layer: it has no repeated span; the scaled form lists none)
+    has_loop_ = c.has("loop") && !form_.gated && !form_.scaled && !form_.dense_parallel;   // (the gated form's depth weights are per layer: it has no repeated span; the other two list none)
+    for (size_t i = 0; i < layers_.size(); ++i) {   // a layer that reads another one's cache rows: an earlier layer with rows of its own, laid out alike
+        const int j = layers_[i].att.kv_from;
+        if (j < 0) continue;
+        const std::string li = "layer " + std::to_string(i);
+        if (j >= (int)i) return fail(NTK_E_FORMAT, li + ": kv_from must name an earlier layer");
+        const WindowMixer &a = layers_[i].att, &b = layers_[(size_t)j].att;
+        if (b.kv_from >= 0) return fail(NTK_E_FORMAT, li + ": kv_from names a layer without keys and values of its own");
+        if (a.kv_heads != b.kv_heads || a.dim != b.dim || a.vdim != b.vdim) return fail(NTK_E_FORMAT, li + ": kv_heads, dim and vdim must equal those of the layer whose keys and values it reads");
+    }
     if (form_.scaled) {   // values are blended with those of the FIRST blending attention layer, which therefore only keeps its own
         const WindowMixer* first = nullptr;
         for (auto& S : layers_) {
@@ -554,19 +604,32 @@ int LayerStackModel::upload_mixer(const ModelFolder& f, const std::string& p, in
     const std::string li = "layer " + std::to_string(i);
     if (L.mixer == kMixWindow) {
         WindowMixer& m = L.att;
-        if (m.gated) LS_TRY(upload_matrix(f, {p + "mix.q", p + "mix.k", p + "mix.v", p + "mix.g"}, W, m.in));
-        else LS_TRY(upload_matrix(f, {p + "mix.q", p + "mix.k", p + "mix.v"}, W, m.in));
+        const bool own = m.kv_from < 0;
+        std::vector<std::string> names = {p + "mix.q"};
+        if (own) { names.push_back(p + "mix.k"); names.push_back(p + "mix.v"); }
+        if (m.gated) names.push_back(p + "mix.g");
+        LS_TRY(upload_matrix(f, names, W, m.in));
         m.k_off = m.heads * m.maps * m.dim;
-        m.v_off = m.k_off + m.kv_heads * m.maps * m.dim;
-        m.g_off = m.v_off + m.kv_heads * m.vdim;
-        const StTensor* tk = f.tensor(p + "mix.k");
-        if (!tk || tk->shape[0] != m.v_off - m.k_off) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.k' does not have kv_heads * maps * dim rows");
+        m.v_off = m.k_off + (own ? m.kv_heads * m.maps * m.dim : 0);
+        m.g_off = m.v_off + (own ? m.kv_heads * m.vdim : 0);
+        if (own && f.tensor(p + "mix.k")->shape[0] != m.v_off - m.k_off) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.k' does not have kv_heads * maps * dim rows");
+        if (form_.whole_qk_norm) {
+            LS_TRY(upload_vector(f, p + "mix.q.norm", m.k_off, &m.q_norm));
+            if (own) LS_TRY(upload_vector(f, p + "mix.k.norm", m.v_off - m.k_off, &m.k_norm));
+        }
+        if (form_.learned_sinks) LS_TRY(upload_vector(f, p + "mix.sink", m.heads, &m.sinks));
         if (m.v_mix && !m.v_source) LS_TRY(read_scalar(f, p + "mix.vmix", &m.v_blend));
-        if (m.in.out_f != m.g_off + (m.gated ? m.heads * m.vdim : 0)) return fail(NTK_E_SHAPE, li + ": the mixer's input projections do not have the configured sizes");
+        if (m.in.out_f != m.g_off + (!m.gated ? 0 : m.head_gate ? m.heads : m.heads * m.vdim)) return fail(NTK_E_SHAPE, li + ": the mixer's input projections do not have the configured sizes");
         const StTensor* tq = f.tensor(p + "mix.q");
         if (!tq || tq->shape[0] != m.k_off) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.q' does not have heads * maps * dim rows");
-        LS_TRY(upload_matrix(f, {p + "mix.o"}, (int64_t)m.heads * m.vdim, m.o));
-        if (m.o.out_f != W) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.o' does not have 'width' rows");
+        const int hv = m.heads * m.vdim;
+        if (form_.dense_parallel && L.has_mlp && hv + L.cff.ff <= kJoinedInputs) {   // the layer's two output products as one
+            LS_TRY(upload_hstack(f, {p + "mix.o", p + "mlp.down"}, L.out));
+            if (L.out.out_f != W || L.out.in_f != hv + L.cff.ff || f.tensor(p + "mix.o")->shape[1] != hv) return fail(NTK_E_SHAPE, li + ": 'mix.o' and 'mlp.down' do not have the configured sizes");
+        } else {
+            LS_TRY(upload_matrix(f, {p + "mix.o"}, hv, m.o));
+            if (m.o.out_f != W) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.o' does not have 'width' rows");
+        }
         m.lambda = 0.0f;
         if (m.maps == 2) {
             // lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff, one number for the layer, in F32
@@ -664,12 +727,12 @@ int LayerStackModel::upload_mixer(const ModelFolder& f, const std::string& p, in
 int LayerStackModel::upload_mlp(const ModelFolder& f, const std::string& p, int i, StackLayer& L) {
     const int W = info_.width;
     const std::string li = "layer " + std::to_string(i);
-    if (L.mlp_kind == kMlpClipped) {
+    if (L.mlp_kind == kMlpUnit) {
         GatedExperts& D = L.cff;
         LS_TRY(upload_matrix(f, {p + "mlp.gate", p + "mlp.up"}, W, D.gate_up));
-        LS_TRY(upload_matrix(f, {p + "mlp.down"}, D.ff, D.down));
+        if (!L.out.ptr) LS_TRY(upload_matrix(f, {p + "mlp.down"}, D.ff, D.down));
         const StTensor* tg = f.tensor(p + "mlp.gate");
-        if (D.gate_up.out_f != 2 * D.ff || !tg || tg->shape[0] != D.ff || D.down.out_f != W) return fail(NTK_E_SHAPE, li + ": feed-forward matrices do not have the configured sizes");
+        if (D.gate_up.out_f != 2 * D.ff || !tg || tg->shape[0] != D.ff || (L.out.ptr ? L.out : D.down).out_f != W) return fail(NTK_E_SHAPE, li + ": feed-forward matrices do not have the configured sizes");
         return NTK_OK;
     }
     if (L.mlp_kind == kMlpDense) {
@@ -751,6 +814,10 @@ int LayerStackModel::load(const std::string& dir, const SeqLoadOptions& opt) {
     else LS_TRY(upload_matrix(f, {"head"}, W, head_));
     if (embed_.out_f != info_.vocab || head_.out_f != info_.vocab) return fail(NTK_E_SHAPE, "embed / head do not have 'vocab' rows");
     LS_TRY(upload_norm(f, "final.norm", final_norm_));
+    if (buckets_ > 0) {
+        LS_TRY(upload_matrix(f, {"bigram"}, W, bigram_));
+        if (bigram_.out_f != (int64_t)buckets_ + 1) return fail(NTK_E_SHAPE, "tensor 'bigram' does not have buckets + 1 rows");
+    }
     if (form_.gated) {
         const StTensor* pt = f.tensor("pos");
         if (!pt || pt->shape.size() != 2 || pt->shape[1] != W) return fail(NTK_E_SHAPE, "tensor 'pos' is not [positions, width]");
@@ -770,6 +837,7 @@ int LayerStackModel::load(const std::string& dir, const SeqLoadOptions& opt) {
     for (size_t i = 0; i < layers_.size(); ++i) LS_TRY(upload_layer(f, (int)i, layers_[i]));
     info_.max_context = opt_.max_context;
     slots_.reset(opt_.slots, opt_.max_context);
+    if (buckets_ > 0) slots_.keep_tokens();
     return alloc_buffers();
 }
 
@@ -801,7 +869,7 @@ int LayerStackModel::alloc_buffers() {
         } else if (L.mixer == kMixWindow) {
             const WindowMixer& m = L.att;
             max_in_ = std::max<int>(max_in_, (int)m.in.out_f);
-            max_hdv_ = std::max(max_hdv_, m.heads * m.vdim);
+            max_hdv_ = std::max(max_hdv_, m.heads * m.vdim + (form_.dense_parallel && L.has_mlp ? L.cff.ff : 0));   // ([joined heads | activations] side by side)
             if (m.vdim > 512) return fail(NTK_E_SHAPE, "vdim up to 512 is supported");
             if (m.v_mix) max_gv_ = std::max(max_gv_, m.kv_heads * m.vdim);
             wsc = std::max(wsc, ntk_window_attention_scratch(chunk_, m.heads, m.maps, m.vdim, opt_.max_context));
@@ -832,7 +900,7 @@ int LayerStackModel::alloc_buffers() {
             if (L.mlp.has_shared) max_sff2_ = std::max(max_sff2_, 2 * L.mlp.shared.ff);
         } else if (L.mlp_kind == kMlpDense && !form_.gated) {
             max_ffn_ = std::max(max_ffn_, L.ffn.ff);
-        } else if (L.mlp_kind == kMlpClipped) {
+        } else if (L.mlp_kind == kMlpUnit) {
             max_ffn_ = std::max(max_ffn_, L.cff.ff);
         }
     }
@@ -851,6 +919,7 @@ int LayerStackModel::alloc_buffers() {
     if (form_.scaled)
         ok = ok && fl(&ff_, C * W) && fl(&zf_, C * std::max(max_ffn_, 1)) && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc) && fl(&rscratch_, rsc) &&
              fl(&cv_, C * std::max(max_conv_, 1)) && fl(&vfirst_, C * std::max(max_gv_, 1));
+    if (form_.dense_parallel) ok = ok && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc);
     want_dev_ = tokens_dev_ ? tokens_dev_ + C : nullptr;   // one staging area: [tokens of a pass | wanted places], filled by ONE stream-ordered copy from pinned memory
     h_stage_ = (int*)nt_hip_malloc_host(2 * C * sizeof(int));
     ok = ok && h_stage_ != nullptr;
@@ -865,7 +934,9 @@ int LayerStackModel::alloc_buffers() {
     for (auto& r : runs_) {
         const StackLayer& L = layers_[(size_t)r.layer];
         const size_t row = (size_t)L.cache_row();
-        if (row) {
+        if (L.att.kv_from >= 0) {
+            r.cache = runs_[(size_t)L.att.kv_from].cache;     // (such a form has no repeated span: run i is layer i)
+        } else if (row) {
             r.cache = (float*)dev_alloc((size_t)opt_.slots * ctx * row * sizeof(float));
             if (!r.cache) return fail(NTK_E_NOMEM, "out of device memory (cache)");
         }
@@ -938,22 +1009,61 @@ int LayerStackModel::run_window(const StackLayer& L, float* cache, int T, int po
     const WindowMixer& m = L.att;
     const int W = info_.width, na = (int)m.in.out_f, hv = m.heads * m.vdim;
     LS_TRY(ntk_dense_linear(a_, na, h1_, W, m.in.ptr, m.in.dtype, T, na, W, 0, stream_));
-    ntk_rotary rot{m.rot_freq, 1.0f, m.rot_dims, form_.rot_halves ? NTK_ROT_HALVES : NTK_ROT_NEIGHBOURS};
+    LS_TRY(window_heads(m, cache, att_, hv, T, pos0));
+    return ntk_dense_linear(mix_, W, att_, hv, m.o.ptr, m.o.dtype, T, W, hv, 0, stream_);
+}
+
+// what lies between the window mixer's two products: norms, rotation and cache rows, then the attention with its gate -> out [T][heads * vdim]
+int LayerStackModel::window_heads(const WindowMixer& m, float* cache, float* out, int ldo, int T, int pos0) {
+    const int na = (int)m.in.out_f;
+    ntk_rotary rot{m.rot_freq, m.rot_mag, m.rot_dims, form_.rot_halves ? NTK_ROT_HALVES : NTK_ROT_NEIGHBOURS};
     ntk_window_prepare_desc pd{};
-    pd.cache = cache; pd.row = m.row(); pd.q = a_; pd.ldq = na; pd.k = a_ + m.k_off; pd.ldk = na; pd.v = a_ + m.v_off; pd.ldv = na;
+    pd.q = a_; pd.ldq = na;
     pd.H = m.heads; pd.G = m.kv_heads; pd.maps = m.maps; pd.dn = m.dim; pd.dv = m.vdim; pd.rot = &rot; pd.temp_every = 1.0; pd.pos0 = pos0; pd.T = T;
+    pd.q_norm = m.q_norm; pd.norm_eps = eps_;
+    if (m.kv_from < 0) {       // (else: the rows another layer wrote for these tokens earlier in the pass)
+        pd.cache = cache; pd.row = m.row(); pd.k = a_ + m.k_off; pd.ldk = na; pd.v = a_ + m.v_off; pd.ldv = na; pd.k_norm = m.k_norm;
+    }
     if (m.v_mix && m.v_source) { pd.v_keep = vfirst_; pd.ld_keep = m.kv_heads * m.vdim; }                 // the first blending layer keeps its values of this pass's tokens
     else if (m.v_mix) { pd.v_other = vfirst_; pd.ld_other = m.kv_heads * m.vdim; pd.v_blend = m.v_blend; }    // the later ones blend with them
     LS_TRY(ntk_window_prepare_ex(&pd, stream_));
     ntk_window_attention_desc d{};
-    d.out = att_; d.ldo = hv; d.q = a_; d.ldq = na; d.cache = cache; d.row = m.row(); d.H = m.heads; d.G = m.kv_heads; d.maps = m.maps; d.dn = m.dim; d.dv = m.vdim;
+    d.out = out; d.ldo = ldo; d.q = a_; d.ldq = na; d.cache = cache; d.row = m.row(); d.H = m.heads; d.G = m.kv_heads; d.maps = m.maps; d.dn = m.dim; d.dv = m.vdim;
     d.pos0 = pos0; d.T = T; d.window = m.window; d.scale = m.scale; d.lambda = m.lambda;
     d.sub_norm = m.maps == 2 ? 1 : 0; d.eps = eps_; d.out_scale = m.maps == 2 ? 1.0f - m.diff : 1.0f;
     d.scratch = wscratch_;
-    d.mask_mode = m.mask_mode; d.softcap = m.softcap; d.sink = m.sink ? 1 : 0;
-    if (m.gated) { d.gate = a_ + m.g_off; d.ldg = na; }     // the elementwise gate rides in the launch that writes the heads' results
-    LS_TRY(ntk_window_attention(&d, stream_));
-    return ntk_dense_linear(mix_, W, att_, hv, m.o.ptr, m.o.dtype, T, W, hv, 0, stream_);
+    d.mask_mode = m.mask_mode; d.softcap = m.softcap; d.sink = m.sink ? 1 : 0; d.keep_first = m.keep_first; d.sinks = m.sinks;
+    if (m.gated) { d.gate = a_ + m.g_off; d.ldg = na; d.head_gate = m.head_gate ? 1 : 0; }     // the gate rides in the launch that writes the heads' results
+    return ntk_window_attention(&d, stream_);
+}
+
+// A layer of the dense parallel form: both sublayers read the stream as it is (decoding: each norm inside its product's launch, the gated unit in the epilogue
+// of its own), then [joined heads | activations] pass both output matrices in ONE product that is added onto the stream.
+int LayerStackModel::dense_parallel_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0) {
+    const WindowMixer& m = L.att;
+    const int W = info_.width, na = (int)m.in.out_f, hv = m.heads * m.vdim, ff = L.has_mlp ? L.cff.ff : 0, no = hv + ff;
+    const bool few = T <= ntk_dense_few_rows();
+    if (!few) LS_TRY(ntk_rmsnorm_offset(h1_, L.norm1.w, ff ? h2_ : nullptr, ff ? L.norm2.w : nullptr, W, x_, W, T, W, eps_, norm_offset_, stream_));
+    ntk_dense_desc d{};
+    d.Y = a_; d.ldy = na; d.X = few ? x_ : h1_; d.ldx = W; d.W = m.in.ptr; d.wdtype = m.in.dtype; d.G = 1; d.row_div = 1; d.T = T; d.N = na; d.K = W;
+    if (few) { d.norm_w = L.norm1.w; d.norm_eps = eps_; d.norm_offset = norm_offset_; }
+    LS_TRY(ntk_dense(&d, stream_));
+    if (ff) {
+        d.W = L.cff.gate_up.ptr; d.wdtype = L.cff.gate_up.dtype; d.N = 2 * ff;
+        if (few) {
+            d.Y = att_ + hv; d.ldy = no; d.norm_w = L.norm2.w;
+            d.glu_ff = ff; d.glu_limit = L.cff.limit; d.glu_alpha = 1.0f; d.glu_up_offset = 0.0f;
+            LS_TRY(ntk_dense(&d, stream_));
+        } else {
+            d.Y = gu2_; d.ldy = 2 * ff; d.X = h2_;
+            LS_TRY(ntk_dense(&d, stream_));
+            LS_TRY(ntk_glu_rows(att_ + hv, no, gu2_, 2 * ff, T, ff, L.cff.limit, 1.0f, 0.0f, 0.0f, stream_));
+        }
+    }
+    LS_TRY(window_heads(m, run.cache + (size_t)slot * opt_.max_context * m.row(), att_, no, T, pos0));
+    if (L.out.ptr) return ntk_dense_linear(x_, W, att_, no, L.out.ptr, L.out.dtype, T, W, no, 1, stream_);
+    LS_TRY(ntk_dense_linear(x_, W, att_, no, m.o.ptr, m.o.dtype, T, W, hv, 1, stream_));
+    return ff ? ntk_dense_linear(x_, W, att_ + hv, no, L.cff.down.ptr, L.cff.down.dtype, T, W, ff, 1, stream_) : NTK_OK;
 }
 
 // the lightning mixer: one product for [q | k | v | gate], the recurrence (silu on the way in), gated RMS norm over the joined heads, output projection -> mix_
@@ -1204,7 +1314,7 @@ int LayerStackModel::parallel_layer(const Run& run, const StackLayer& L, int slo
     return ntk_residual_add(x_, mix_, nullptr, T * W, stream_);
 }
 
-int LayerStackModel::portion(int slot, const int* tokens_dev, int T, int pos0, const int* want_dev, int n_want, float* logits_out) {
+int LayerStackModel::portion(int slot, const int* tokens_dev, int prev_token, int T, int pos0, const int* want_dev, int n_want, float* logits_out) {
     const int W = info_.width;
     // (the embedding is kept beside the stream only where a repeated span is entered through a projection of both)
     const bool keep_embedding = has_loop_ && form_.loop_projection;
@@ -1214,6 +1324,8 @@ int LayerStackModel::portion(int slot, const int* tokens_dev, int T, int pos0, c
                                    embed_norm_.alpha, stream_));
         const NormW& n1 = layers_[(size_t)runs_[0].layer].norm1;
         LS_TRY(ntk_dyt(h1_, W, x_, W, n1.w, n1.b, n1.alpha, T, W, stream_));
+    } else if (buckets_ > 0) {
+        LS_TRY(ntk_embed_bigram(x_, embed_.ptr, bigram_.ptr, embed_.dtype, tokens_dev, prev_token, pos0, T, info_.vocab, W, embed_scale_, buckets_, mul_prev_, mul_cur_, stream_));
     } else
     LS_TRY(ntk_embed_dense_scaled(keep_embedding ? x0_ : x_, embed_.ptr, embed_.dtype, tokens_dev, T, info_.vocab, W, embed_scale_, stream_));
     bool x_is_x0 = keep_embedding;   // until the first layer run writes x_
@@ -1235,6 +1347,8 @@ int LayerStackModel::portion(int slot, const int* tokens_dev, int T, int pos0, c
         } else if (form_.sequential) {
             LS_TRY(sequential_layer(run, L, slot, T, pos0));
             if (r + 1 == runs_.size() || (capture_ && capture_buf_)) LS_TRY(settle(T));
+        } else if (form_.dense_parallel) {
+            LS_TRY(dense_parallel_layer(run, L, slot, T, pos0));
         } else {
             LS_TRY(parallel_layer(run, L, slot, T, pos0));
         }
@@ -1300,10 +1414,12 @@ float* LayerStackModel::forward(int slot, const int* tokens, int n, const int* w
         const int nw = w1 - done_want;
         if (nw > 0) memcpy(h_stage_ + chunk_, rel.data(), (size_t)nw * sizeof(int));
         if (ntk_memcpy_h2d_async(tokens_dev_, h_stage_, (size_t)(nw > 0 ? chunk_ + nw : T) * sizeof(int), stream_) != NTK_OK) { err_ = "forward: the copy of the tokens failed"; return nullptr; }
-        const int st = portion(slot, tokens_dev_, T, pos0 + at, want_dev_, w1 - done_want, logits_ + (size_t)done_want * info_.vocab);
+        const int prev_token = at > 0 ? tokens[at - 1] : pos0 > 0 ? slots_.token(slot, pos0 - 1) : 0;
+        const int st = portion(slot, tokens_dev_, prev_token, T, pos0 + at, want_dev_, w1 - done_want, logits_ + (size_t)done_want * info_.vocab);
         if (st != NTK_OK) { if (err_.empty()) err_ = std::string("forward: ") + ntk_status_string(st); return nullptr; }
         done_want = w1;
     }
+    slots_.record(slot, pos0, tokens, n);
     slots_.set_length(slot, pos0 + n);
     last_rows_ = n_want;
     return logits_;

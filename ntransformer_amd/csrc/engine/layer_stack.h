@@ -3,6 +3,9 @@
 // output norm + head.  A family fixes the FORM of a layer (StackForm):
 //   parallel     x += mixer(norm1 x) + ff(norm2 x), RMS norms whose weight is stored around zero; the repeated span is entered through a projection
 //                of [stream ; embedding]                                                                                   -- "Fabolorn"
+//                or (dense_parallel) with plain norm weights, grouped-query attention and one dense gated unit per layer, whose two last products are ONE
+//                product over [joined heads | activations] added onto the stream; scaled embedding plus a row picked by the token and the one before it
+//                                                                                                                           -- "Zalazen"
 //   sequential   x += norm1b(mixer(conv(norm1 x))), then x += norm2b(ff(conv(norm2 x))): layer norms with weight and bias before and after every
 //                sublayer, a short causal convolution added to every sublayer's input (its last inputs are part of a sequence's state), scaled
 //                embedding and logits                                                                                       -- "Nizorax"
@@ -28,11 +31,15 @@
 //                 in the softmax, values blended with those of the first such layer and an elementwise output gate (the same WindowMixer and kernels with
 //                 other parameters), "latent_attention" pairs rotated entries half against half and gates per head, and "delta" is the delta rule with
 //                 one decay and one write strength per head over unit queries and keys that went through a short convolution (GatedDeltaMixer);
+//                 in the dense parallel form "attention" is grouped-query attention over a sliding window beside which a sequence's first positions stay
+//                 visible, with queries and keys normed over their whole projection, half-split rotation with blended frequencies, a learned sink and one gate
+//                 per head, and optionally the keys and values of an EARLIER layer instead of its own (the same WindowMixer and kernels);
 //   feed-forward  kind "moe": routed gated experts + an optional shared expert (MoeFeedForward: softmax or sigmoid scores, optional expert groups,
 //                 clipped or plain gated units); kind "dense": up, polynomial activation with unit-norm terms, down (DenseFeedForward), or in the
 //                 gated form a gated unit with the tanh form of gelu (GatedFeedForward), in the scaled form the clipped gated unit of the experts as one
-//                 dense unit (GatedExperts with one member).
-// What a sequence holds per layer run: cache rows per position (attention kinds), a recurrent state (lightning, gla, delta rules), the convolutions' last inputs.
+//                 dense unit, in the dense parallel form the plain one (GatedExperts with one member).
+// What a sequence holds per layer run: cache rows per position (attention kinds; none where a layer reads another one's), a recurrent state (lightning, gla, delta
+// rules), the convolutions' last inputs; and per slot its token ids where the embedding reads the token before.
 #pragma once
 #include <string>
 #include <vector>
@@ -77,11 +84,17 @@ struct WindowMixer {                  // grouped-query attention, sliding window
     double* rot_freq = nullptr;       // device [rot_dims / 2]
     int mask_mode = NTK_MASK_SLIDING; // what `window` means: a sliding window or chunks of the sequence
     float softcap = 0.0f;             // > 0: scores pass cap * tanh(. / cap)
+    int keep_first = 0;               // positions that stay visible beside a sliding window
     bool sink = false;                // one more exp(0) in every softmax's denominator
-    bool gated = false;               // elementwise sigmoid gate on the joined heads (its rows sit behind v in `in`)
+    float* sinks = nullptr;           // ... or exp(sinks[h]), F32 [heads]
+    bool gated = false;               // sigmoid gate on the joined heads (its rows sit behind v in `in`), elementwise or one number per head
+    bool head_gate = false;
+    float *q_norm = nullptr, *k_norm = nullptr;   // F32 [heads * dim], [kv_heads * dim]: RMS norm over the whole projection, ahead of the rotation
+    float rot_mag = 1.0f;
+    int kv_from = -1;                 // >= 0: this layer has no keys and values of its own, it reads the cache rows of that layer
     bool v_mix = false, v_source = false;   // values blended with those of the first such layer (v_source: this IS that layer, it only keeps them)
     float v_blend = 0.0f;
-    DenseW in;                        // rows [q | k | v (| gate)] of one product over the mixer's input
+    DenseW in;                        // rows [q | k | v (| gate)] of one product over the mixer's input (kv_from: [q | gate])
     int k_off = 0, v_off = 0, g_off = 0;
     DenseW o;
     int row() const { return kv_heads * (maps * dim + vdim); }
@@ -183,7 +196,7 @@ struct DenseFeedForward {             // down(act(up h)), act = a N(z) + b N(z^2
 struct NormW { float* w = nullptr; float* b = nullptr; float alpha = 0.0f; };   // b: layer norm with bias (sequential form) / dynamic tanh with its alpha (gated form); none: RMS norm, weight around zero
 
 enum MixerKind { kMixLatent = 0, kMixWindow = 1, kMixLightning = 2, kMixGla = 3, kMixParallel = 4, kMixGatedDelta = 5 };
-enum MlpKind { kMlpNone = 0, kMlpMoe = 1, kMlpDense = 2, kMlpClipped = 3 };
+enum MlpKind { kMlpNone = 0, kMlpMoe = 1, kMlpDense = 2, kMlpUnit = 3 };   // (unit: one dense gated unit)
 
 struct StackLayer {
     std::string type;
@@ -197,7 +210,8 @@ struct StackLayer {
     GlaMixer gla;
     ParallelMixer par;
     GatedDeltaMixer gdl;
-    GatedExperts cff;                       // scaled form: one dense clipped gated unit
+    GatedExperts cff;                       // scaled and dense parallel form: one dense gated unit
+    DenseW out;                             // dense parallel form: [width][heads * vdim + ff], both output products side by side (none: att.o and cff.down apart)
     GatedFeedForward gff;
     float *rg1_b = nullptr, *rg2_b = nullptr;   // gated form: biases of the residual gates, F32 [width]
     float* depth = nullptr;                 // gated form: weights of the layer results so far (embedding first), device F32 [layer + 2]
@@ -217,6 +231,11 @@ struct StackForm {
     bool sequential = false;          // see the head of this file
     bool gated = false;               // ...
     bool scaled = false;              // ... (none of the three: the parallel form)
+    bool dense_parallel = false;      // the parallel form with plain norm weights, window attention and one dense gated unit
+    bool blended_rotation = false;    // an attention layer's rotary scaling: a ramp over the pair index, with a magnitude (else by wavelength)
+    bool learned_sinks = false;       // an attention layer's softmax has a learned sink per head
+    bool attention_head_gate = false; // its output gate is one number per head
+    bool whole_qk_norm = false;       // its queries and keys are normed over the whole projection
     // the scaled form's mechanisms: what its design fixes about them
     bool mask_chunks = false;         // an attention layer's mask.size is a chunk size (else a sliding window)
     bool attention_sink = false;      // its softmax has a sink
@@ -281,9 +300,11 @@ private:
     int upload_matrix(const ModelFolder& f, const std::vector<std::string>& names, int64_t in_f, DenseW& out, int count = 1);
     int alloc_buffers();
     void* dev_alloc(size_t bytes);
-    int portion(int slot, const int* tokens_dev, int T, int pos0, const int* want_dev, int n_want, float* logits_out);
+    int portion(int slot, const int* tokens_dev, int prev_token, int T, int pos0, const int* want_dev, int n_want, float* logits_out);
     int run_mixer(const StackLayer& L, float* cache, int T, int pos0, bool normed_input = false);
     int run_window(const StackLayer& L, float* cache, int T, int pos0);
+    int window_heads(const WindowMixer& m, float* cache, float* out, int ldo, int T, int pos0);
+    int dense_parallel_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0);
     int run_lightning(const StackLayer& L, float* state, int T, int pos0);
     int run_moe(const StackLayer& L, int T, bool into_stream);
     int run_dense_ff(const StackLayer& L, int T);
@@ -310,6 +331,9 @@ private:
     std::vector<Run> runs_;
     bool has_loop_ = false;
     DenseW embed_, head_, loop_in_, pos_;   // pos_: a learned vector per position (gated form)
+    DenseW bigram_;                   // [buckets + 1][width]: the row picked by (previous token, token); the last one is a first token's
+    int buckets_ = 0;                 // 0: no such table
+    long long mul_prev_ = 0, mul_cur_ = 0;
     NormW embed_norm_;
     int n_positions_ = 0;             // rows of the position table
     NormW final_norm_;

@@ -73,9 +73,16 @@ public:
     int length(int s) const { return live(s) ? len_[(size_t)s] : -1; }
     bool release(int s) { if (!live(s)) return false; len_[(size_t)s] = -1; return true; }
     bool set_length(int s, int n) { if (!live(s) || n < 0 || n > cap_) return false; len_[(size_t)s] = n; return true; }
+    // for families whose step reads earlier TOKENS themselves: the ids a slot was given, by position (host memory; a slot cut back keeps the ones before the cut)
+    void keep_tokens() { tokens_.assign(len_.size() * (size_t)cap_, 0); }
+    void record(int s, int at, const int* ids, int n) {
+        if (tokens_.empty()) return;
+        for (int i = 0; i < n; ++i) tokens_[(size_t)s * cap_ + at + i] = ids[i];
+    }
+    int token(int s, int at) const { return tokens_.empty() ? 0 : tokens_[(size_t)s * cap_ + at]; }
 
 private:
-    std::vector<int> len_;
+    std::vector<int> len_, tokens_;
     int cap_ = 0;
 };
 

@@ -23,6 +23,26 @@ __global__ __launch_bounds__(256) void embed_dense_kernel(float* out, const TT* 
     }
 }
 
+template <typename TT> __device__ __forceinline__ float table_value(const TT* row, int i) {
+    if constexpr (sizeof(TT) == 2) return __uint_as_float((uint32_t)row[i] << 16); else return row[i];
+}
+// the token's row plus a row picked by the token and the one before it
+template <typename TT>
+__global__ __launch_bounds__(256) void embed_bigram_kernel(float* out, const TT* table, const TT* bigram, const int* tokens, int prev, int pos0, int vocab, int width,
+                                                           float scale, int buckets, long long mul_prev, long long mul_cur) {
+    const int t = blockIdx.x, tok = tokens[t];
+    float* o = out + (long long)t * width;
+    const bool ok = tok >= 0 && tok < vocab;
+    long long r = buckets;                                   // a sequence's first token
+    if (pos0 + t > 0) {
+        r = ((long long)(t > 0 ? tokens[t - 1] : prev) * mul_prev + (long long)tok * mul_cur) % buckets;
+        if (r < 0) r += buckets;
+    }
+    const TT* row = table + (long long)(ok ? tok : 0) * width;
+    const TT* two = bigram + r * width;
+    for (int i = threadIdx.x; i < width; i += 256) o[i] = fmaf(ok ? table_value(row, i) : 0.0f, scale, table_value(two, i));
+}
+
 __global__ __launch_bounds__(256) void rmsnorm_offset_kernel(float* y1, const float* w1, float* y2, const float* w2, int ldy, const float* x, int ldx, int n,
                                                              float eps, float offset) {
     __shared__ float red[16];
@@ -212,6 +232,21 @@ int ntk_embed_dense_scaled(float* out, const void* table, int tdtype, const int*
     if (tdtype == NTK_DT_BF16) hipLaunchKernelGGL(embed_dense_kernel<uint16_t>, dim3(T), dim3(256), 0, resolve_stream(stream), out, (const uint16_t*)table, tokens, vocab, width, scale);
     else if (tdtype == NTK_DT_F32) hipLaunchKernelGGL(embed_dense_kernel<float>, dim3(T), dim3(256), 0, resolve_stream(stream), out, (const float*)table, tokens, vocab, width, scale);
     else return NTK_E_DTYPE;
+    return last_launch_status();
+}
+
+int ntk_embed_bigram(float* out, const void* table, const void* bigram, int tdtype, const int* tokens, int prev, int pos0, int T, int vocab, int width, float scale,
+                     int buckets, long long mul_prev, long long mul_cur, void* stream) {
+    if (!out || !table || !bigram || !tokens) return NTK_E_NULL;
+    if (tdtype != NTK_DT_BF16 && tdtype != NTK_DT_F32) return NTK_E_DTYPE;
+    if (T < 0 || vocab <= 0 || width <= 0 || pos0 < 0 || buckets <= 0) return NTK_E_SHAPE;
+    if (T == 0) return NTK_OK;
+    if (tdtype == NTK_DT_BF16)
+        hipLaunchKernelGGL(embed_bigram_kernel<uint16_t>, dim3(T), dim3(256), 0, resolve_stream(stream), out, (const uint16_t*)table, (const uint16_t*)bigram, tokens, prev,
+                           pos0, vocab, width, scale, buckets, mul_prev, mul_cur);
+    else
+        hipLaunchKernelGGL(embed_bigram_kernel<float>, dim3(T), dim3(256), 0, resolve_stream(stream), out, (const float*)table, (const float*)bigram, tokens, prev, pos0,
+                           vocab, width, scale, buckets, mul_prev, mul_cur);
     return last_launch_status();
 }
 

@@ -189,14 +189,14 @@ __global__ __launch_bounds__(kGroupThreads) void moe_group_kernel(int* offsets, 
     }
 }
 
-__global__ void clipped_glu_kernel(float* a, const float* gu, int ldgu, int ff, float limit, float alpha, float cubic, float up_offset) {
+__global__ void clipped_glu_kernel(float* a, int lda, const float* gu, int ldgu, int ff, float limit, float alpha, float cubic, float up_offset) {
     const long long r = blockIdx.y;
     const int f = blockIdx.x * blockDim.x + threadIdx.x;
     if (f >= ff) return;
     const float g = fminf(gu[r * ldgu + f], limit);
     const float u = fminf(fmaxf(gu[r * ldgu + ff + f], -limit), limit);
     const float z = cubic != 0.0f ? fmaf(cubic * g * g, g, g) : g;
-    a[r * ff + f] = g * (1.0f / (1.0f + expf(-alpha * z))) * (u + up_offset);
+    a[r * lda + f] = g * (1.0f / (1.0f + expf(-alpha * z))) * (u + up_offset);
 }
 
 template <bool ADD>
@@ -250,18 +250,18 @@ int ntk_clipped_glu(float* a, const float* gu, int rows, int ff, float limit, fl
 }
 
 int ntk_glu(float* a, const float* gu, int rows, int ff, float limit, float alpha, float up_offset, void* stream) {
-    if (!a || !gu) return NTK_E_NULL;
-    if (rows < 0 || ff <= 0) return NTK_E_SHAPE;
-    if (rows == 0) return NTK_OK;
-    hipLaunchKernelGGL(clipped_glu_kernel, dim3((ff + 255) / 256, rows), dim3(256), 0, resolve_stream(stream), a, gu, 2 * ff, ff, limit, alpha, 0.0f, up_offset);
-    return last_launch_status();
+    return ntk_glu_rows(a, ff, gu, 2 * ff, rows, ff, limit, alpha, 0.0f, up_offset, stream);
 }
 
 int ntk_glu_cubic(float* a, const float* gu, int ldgu, int rows, int ff, float limit, float alpha, float cubic, float up_offset, void* stream) {
+    return ntk_glu_rows(a, ff, gu, ldgu, rows, ff, limit, alpha, cubic, up_offset, stream);
+}
+
+int ntk_glu_rows(float* a, int lda, const float* gu, int ldgu, int rows, int ff, float limit, float alpha, float cubic, float up_offset, void* stream) {
     if (!a || !gu) return NTK_E_NULL;
-    if (rows < 0 || ff <= 0 || ldgu < 2 * ff) return NTK_E_SHAPE;
+    if (rows < 0 || ff <= 0 || ldgu < 2 * ff || lda < ff) return NTK_E_SHAPE;
     if (rows == 0) return NTK_OK;
-    hipLaunchKernelGGL(clipped_glu_kernel, dim3((ff + 255) / 256, rows), dim3(256), 0, resolve_stream(stream), a, gu, ldgu, ff, limit, alpha, cubic, up_offset);
+    hipLaunchKernelGGL(clipped_glu_kernel, dim3((ff + 255) / 256, rows), dim3(256), 0, resolve_stream(stream), a, lda, gu, ldgu, ff, limit, alpha, cubic, up_offset);
     return last_launch_status();
 }
 

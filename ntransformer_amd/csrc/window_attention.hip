@@ -1,8 +1,9 @@
 // window_attention.hip -- grouped-query softmax attention over a cache of rotated keys and values: causal, optional sliding window, one or two score
 // maps per head over the same values (two maps: the differential pair out = a_0 - lambda * a_1), optional unit norm of every head's output, optional
 // learned bias by bucketed distance on the scaled score (a table of distances -> buckets, a table of buckets x heads), optional cap on the score
-// (cap * tanh(score / cap)), optional sink (a key of score 0 without a value in every softmax), and instead of the sliding window a mask of chunks
-// (a query sees the keys of its own chunk of `window` positions, counted from position 0, up to itself).
+// (cap * tanh(score / cap)), optional sink (a key without a value in every softmax: of score 0, or of a learned score per head), optional gate on the output
+// (element by element or one number per head); beside the sliding window the first `keep_first` positions can stay visible for ever, and instead of it there is a
+// mask of chunks (a query sees the keys of its own chunk of `window` positions, counted from position 0, up to itself).
 //
 // Cache row of a position: [G][maps][dn] rotated keys | [G][dv] values, F32.  Scores, softmax, weights and sums are F32 on the vector units.
 // A workgroup owns 16 (token, head) rows of ONE key/value head -- consecutive tokens times the heads that share it, so a key or value slab that was
@@ -16,55 +17,81 @@
 namespace ntk {
 
 // one workgroup per token: q rotated in place, k rotated into the cache row, v copied behind.  Angles in double (position times frequency), applied in F32.
-// Optional: what the projections left to their consumer -- bias vectors on q, k and v, and a query temperature that grows with the position.
-__global__ __launch_bounds__(256) void window_prepare_kernel(float* cache, int row, float* q, int ldq, const float* k, int ldk, const float* v, int ldv, int nq, int nk,
-                                                             int dn, int nv, const double* freq, float mag, int dims, int pos0, const float* qb, const float* kb,
-                                                             const float* vb, float temp_coef, double temp_every, int halves, const float* v_other, int ld_other,
-                                                             float v_blend, float* v_keep, int ld_keep) {
+// Optional: what the projections left to their consumer -- bias vectors on q, k and v, and a query temperature that grows with the position --, and an RMS norm
+// over the token's WHOLE q (and whole k) ahead of the rotation.  k == NULL: queries only (a layer that reads another layer's cache rows).
+struct PrepareArgs {
+    float* cache; int row;
+    float* q; int ldq; const float* k; int ldk; const float* v; int ldv;
+    int nq, nk, dn, nv;                      // vectors of dn entries in q and in k (heads x maps), value entries
+    const double* freq; float mag; int dims, halves, pos0;
+    const float *qb, *kb, *vb; float temp_coef; double temp_every;
+    const float* v_other; int ld_other; float v_blend; float* v_keep; int ld_keep;
+    const float *q_norm, *k_norm; float norm_eps;
+};
+
+template <int NT>
+__global__ __launch_bounds__(NT) void window_prepare_kernel(const PrepareArgs a) {
     extern __shared__ float cs[];   // [dims / 2] cos, [dims / 2] sin
-    const int t = blockIdx.x, pos = pos0 + t;
-    const int half = dims / 2;
-    if (qb || temp_coef != 0.0f) {     // (uniform over the launch) q = (q + bias) * temperature, ahead of the rotation: a thread rewrites its own entries
-        float* qt0 = q + (long long)t * ldq;
-        const float temp = temp_coef != 0.0f ? 1.0f + temp_coef * logf((float)floor((double)(pos + 1) / temp_every) + 1.0f) : 1.0f;
-        for (int j = threadIdx.x; j < nq * dn; j += 256) qt0[j] = (qt0[j] + (qb ? qb[j] : 0.0f)) * temp;
+    const int t = blockIdx.x, pos = a.pos0 + t, dn = a.dn;
+    const int half = a.dims / 2;
+    float* qt = a.q + (long long)t * a.ldq;
+    const float* kt = a.k ? a.k + (long long)t * a.ldk : nullptr;
+    if (a.qb || a.temp_coef != 0.0f) {     // (uniform over the launch) q = (q + bias) * temperature, ahead of the rotation: a thread rewrites its own entries
+        const float temp = a.temp_coef != 0.0f ? 1.0f + a.temp_coef * logf((float)floor((double)(pos + 1) / a.temp_every) + 1.0f) : 1.0f;
+        for (int j = threadIdx.x; j < a.nq * dn; j += NT) qt[j] = (qt[j] + (a.qb ? a.qb[j] : 0.0f)) * temp;
         __syncthreads();
     }
-    for (int i = threadIdx.x; i < half; i += 256) {
-        const double a = (double)pos * freq[i];
-        cs[i] = (float)(cos(a) * (double)mag);
-        cs[half + i] = (float)(sin(a) * (double)mag);
+    for (int i = threadIdx.x; i < half; i += NT) {
+        const double ang = (double)pos * a.freq[i];
+        cs[i] = (float)(cos(ang) * (double)a.mag);
+        cs[half + i] = (float)(sin(ang) * (double)a.mag);
+    }
+    float qs = 1.0f, ks = 1.0f;            // one over the root mean square of the whole q / k
+    if (a.q_norm || a.k_norm) {            // (uniform over the launch)
+        __shared__ float red[16];
+        float sq = 0.0f, sk = 0.0f;
+        if (a.q_norm) for (int j = threadIdx.x; j < a.nq * dn; j += NT) sq = fmaf(qt[j], qt[j], sq);
+        if (a.k_norm && kt)
+            for (int j = threadIdx.x; j < a.nk * dn; j += NT) { const float x = kt[j] + (a.kb ? a.kb[j] : 0.0f); sk = fmaf(x, x, sk); }
+        if (a.q_norm) qs = 1.0f / sqrtf(block_sum(sq, red) / (float)(a.nq * dn) + a.norm_eps);
+        if (a.k_norm && kt) ks = 1.0f / sqrtf(block_sum(sk, red) / (float)(a.nk * dn) + a.norm_eps);
     }
     __syncthreads();
-    float* dst = cache + (long long)pos * row;
-    float* qt = q + (long long)t * ldq;
-    const float* kt = k + (long long)t * ldk;
-    const float* vt = v + (long long)t * ldv;
-    const int pair = halves ? half : 1, step = halves ? 1 : 2;   // pair i = entries (i * step, i * step + pair)
-    for (int j = threadIdx.x; j < nq * half; j += 256) {       // nq = heads x maps vectors of dn
-        float* p = qt + (j / half) * dn + step * (j % half);
-        float ra, rb;
-        rope_rotate(p[0], p[pair], cs[j % half], cs[half + j % half], ra, rb);
-        p[0] = ra;
-        p[pair] = rb;
-    }
-    for (int j = threadIdx.x; j < nk * half; j += 256) {
+    auto q_at = [&](int o) { return a.q_norm ? qt[o] * qs * a.q_norm[o] : qt[o]; };
+    auto k_at = [&](int o) { const float x = kt[o] + (a.kb ? a.kb[o] : 0.0f); return a.k_norm ? x * ks * a.k_norm[o] : x; };
+    const int pair = a.halves ? half : 1, step = a.halves ? 1 : 2;   // pair i = entries (i * step, i * step + pair)
+    const int rest = dn - a.dims;
+    for (int j = threadIdx.x; j < a.nq * half; j += NT) {       // nq = heads x maps vectors of dn
         const int o = (j / half) * dn + step * (j % half);
         float ra, rb;
-        rope_rotate(kt[o] + (kb ? kb[o] : 0.0f), kt[o + pair] + (kb ? kb[o + pair] : 0.0f), cs[j % half], cs[half + j % half], ra, rb);
+        rope_rotate(q_at(o), q_at(o + pair), cs[j % half], cs[half + j % half], ra, rb);
+        qt[o] = ra;
+        qt[o + pair] = rb;
+    }
+    if (a.q_norm)
+        for (int j = threadIdx.x; j < a.nq * rest; j += NT) {
+            const int o = (j / rest) * dn + a.dims + j % rest;
+            qt[o] = q_at(o);
+        }
+    if (!kt) return;
+    float* dst = a.cache + (long long)pos * a.row;
+    const float* vt = a.v + (long long)t * a.ldv;
+    for (int j = threadIdx.x; j < a.nk * half; j += NT) {
+        const int o = (j / half) * dn + step * (j % half);
+        float ra, rb;
+        rope_rotate(k_at(o), k_at(o + pair), cs[j % half], cs[half + j % half], ra, rb);
         dst[o] = ra;
         dst[o + pair] = rb;
     }
-    const int rest = dn - dims;
-    for (int j = threadIdx.x; j < nk * rest; j += 256) {
-        const int o = (j / rest) * dn + dims + j % rest;
-        dst[o] = kt[o] + (kb ? kb[o] : 0.0f);
+    for (int j = threadIdx.x; j < a.nk * rest; j += NT) {
+        const int o = (j / rest) * dn + a.dims + j % rest;
+        dst[o] = k_at(o);
     }
-    for (int j = threadIdx.x; j < nv; j += 256) {
-        float vv = vt[j] + (vb ? vb[j] : 0.0f);
-        if (v_keep) v_keep[(long long)t * ld_keep + j] = vv;
-        if (v_other) vv = fmaf(v_blend, v_other[(long long)t * ld_other + j], (1.0f - v_blend) * vv);
-        dst[nk * dn + j] = vv;
+    for (int j = threadIdx.x; j < a.nv; j += NT) {
+        float vv = vt[j] + (a.vb ? a.vb[j] : 0.0f);
+        if (a.v_keep) a.v_keep[(long long)t * a.ld_keep + j] = vv;
+        if (a.v_other) vv = fmaf(a.v_blend, a.v_other[(long long)t * a.ld_other + j], (1.0f - a.v_blend) * vv);
+        dst[a.nk * dn + j] = vv;
     }
 }
 
@@ -78,7 +105,9 @@ struct WinArgs {
     int splits; float* scratch;       // splits > 1: states [T * H][splits][maps][2 + dv]
     const float* rel; const int* bucket_of; int n_dist;   // rel != NULL: rel[bucket_of[min(distance, n_dist - 1)] * H + head] joins the scaled score
     int chunks; float softcap; int sink;                  // chunks != 0: `window` is a chunk size
-    const float* gate; int ldg;                           // gate != NULL: out[t][h][c] *= sigmoid(gate[t * ldg + h * dv + c])
+    const float* gate; int ldg, head_gate;                // gate != NULL: out[t][h][c] *= sigmoid(gate[t * ldg + h * dv + c]), or gate[t * ldg + h] with head_gate
+    int keep;                                             // positions 0 .. keep - 1 stay visible behind the sliding window
+    const float* sinks;                                   // the sink's score per head (NULL with `sink`: 0)
 };
 
 // first key a query at position p sees
@@ -89,9 +118,14 @@ __device__ __forceinline__ int first_visible(int p, int window, int chunks) {
 
 constexpr int WROWS = 16, WQPW = 4, WKCH = 64, WSLAB = 64, WMAXC = 8;   // dv <= WMAXC * WSLAB
 
+// the gate of row (t, h): its first entry and the distance to the next column's (0: one gate for the head)
+__device__ __forceinline__ const float* gate_of(const WinArgs& a, int t, int h) {
+    return a.gate ? a.gate + (long long)t * a.ldg + (a.head_gate ? h : h * a.dv) : nullptr;
+}
+
 // the differential pair, the unit norm and the scale on a row whose lanes hold columns c * 64 + lane
 template <int M>
-__device__ __forceinline__ void finish_row(float (&a)[M][WMAXC], int lane, int dv, float lambda, int sub_norm, float eps, float out_scale, float* o, const float* gate) {
+__device__ __forceinline__ void finish_row(float (&a)[M][WMAXC], int lane, int dv, float lambda, int sub_norm, float eps, float out_scale, float* o, const float* gate, int gate_step) {
     float r[WMAXC];
     float ss = 0.0f;
 #pragma unroll
@@ -106,7 +140,7 @@ __device__ __forceinline__ void finish_row(float (&a)[M][WMAXC], int lane, int d
     if (sub_norm) mul = out_scale / sqrtf(wave_sum(ss) / (float)dv + eps);
 #pragma unroll
     for (int c = 0; c < WMAXC; ++c)
-        if (c * WSLAB + lane < dv) o[c * WSLAB + lane] = gate ? r[c] * mul / (1.0f + expf(-gate[c * WSLAB + lane])) : r[c] * mul;
+        if (c * WSLAB + lane < dv) o[c * WSLAB + lane] = gate ? r[c] * mul / (1.0f + expf(-gate[(c * WSLAB + lane) * gate_step])) : r[c] * mul;
 }
 
 template <int M>
@@ -123,6 +157,9 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
     const int pmin = a.pos0 + row0 / R, pmax = a.pos0 + last / R;
     const int jlo = first_visible(pmin, a.window, a.chunks);
     const int jhi = pmax;   // inclusive
+    // the keys walked: positions 0 .. kept - 1 (those of the kept first ones that lie before the window), then jlo .. jhi; key number i of the walk is position
+    // i, or i + skip from `kept` on
+    const int kept = min(a.keep, jlo), skip = jlo - kept, n_keys = kept + jhi - jlo + 1;
     // queries into LDS
     for (int e0 = threadIdx.x; e0 < WROWS * M * DNP; e0 += 256 * 4) {     // (four of a thread's entries asked for before the first is stored)
         float qv[4];
@@ -143,21 +180,23 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
         const int rho = row0 + wave * WQPW + i;
         rpos[i] = rho < n_rows ? a.pos0 + rho / R : -1;
         rhead[i] = g * R + rho % R;
-        // the sink is a key of score 0 without a value: the running maximum and sum start from it (in the first part only when the keys are split)
-        const bool sunk = a.sink && (a.splits <= 1 || blockIdx.z == 0);
+        // the sink is a key without a value: the running maximum and sum start from it (in the first part only when the keys are split)
+        const bool sunk = (a.sink || a.sinks) && (a.splits <= 1 || blockIdx.z == 0);
+        const float sink_score = a.sinks ? a.sinks[rhead[i]] : 0.0f;
 #pragma unroll
         for (int m = 0; m < M; ++m) {
-            mx[m][i] = sunk ? 0.0f : -INFINITY; l[m][i] = sunk ? 1.0f : 0.0f;
+            mx[m][i] = sunk ? sink_score : -INFINITY; l[m][i] = sunk ? 1.0f : 0.0f;
 #pragma unroll
             for (int c = 0; c < WMAXC; ++c) acc[m][i][c] = 0.0f;
         }
     }
     const int vbase = a.G * M * a.dn + g * a.dv;
     int chunk = 0;
-    for (int j0 = jlo; j0 <= jhi; j0 += WKCH, ++chunk) {
+    for (int i0 = 0; i0 < n_keys; i0 += WKCH, ++chunk) {
         if (a.splits > 1 && chunk % a.splits != (int)blockIdx.z) continue;     // (uniform over the workgroup)
-        const int nk = min(WKCH, jhi + 1 - j0);
-        const int j = j0 + lane;
+        const int nk = min(WKCH, n_keys - i0);
+        auto key_pos = [&](int k) { return i0 + k + (i0 + k >= kept ? skip : 0); };   // position of the chunk's key k
+        const int j = key_pos(lane);
 #pragma unroll
         for (int m = 0; m < M; ++m) {
             float s[WQPW];
@@ -168,12 +207,12 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
                 const int nd = min(WSLAB, a.dn - d0);
                 __syncthreads();
                 {   // thread -> (key wave + 4 u, entry lane): the sixteen requests of a thread in flight before the first is stored
-                    const float* src = a.cache + (long long)j0 * a.row + (g * M + m) * a.dn + d0 + lane;
+                    const float* src = a.cache + (g * M + m) * a.dn + d0 + lane;
                     float v[16];
 #pragma unroll
                     for (int u = 0; u < 16; ++u) {
                         const int k = wave + 4 * u;
-                        v[u] = (k < nk && lane < nd) ? src[(long long)k * a.row] : 0.0f;
+                        v[u] = (k < nk && lane < nd) ? src[(long long)key_pos(k) * a.row] : 0.0f;
                     }
 #pragma unroll
                     for (int u = 0; u < 16; ++u) Sl[(wave + 4 * u) * (WSLAB + 1) + lane] = v[u];
@@ -192,7 +231,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
             // ---- online softmax of map m, weights to LDS
 #pragma unroll
             for (int i = 0; i < WQPW; ++i) {
-                const bool vis = lane < nk && rpos[i] >= 0 && j <= rpos[i] && j >= first_visible(rpos[i], a.window, a.chunks);
+                const bool vis = lane < nk && rpos[i] >= 0 && j <= rpos[i] && (j >= first_visible(rpos[i], a.window, a.chunks) || j < a.keep);
                 float sv = vis ? s[i] * a.scale : -INFINITY;
                 if (a.rel && vis) sv += a.rel[(long long)a.bucket_of[min(rpos[i] - j, a.n_dist - 1)] * a.H + rhead[i]];
                 if (a.softcap > 0.0f && vis) sv = a.softcap * tanhf(sv / a.softcap);
@@ -215,12 +254,12 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
                 const int nvv = min(WSLAB, a.dv - v0);
                 __syncthreads();
                 {
-                    const float* src = a.cache + (long long)j0 * a.row + vbase + v0 + lane;
+                    const float* src = a.cache + vbase + v0 + lane;
                     float v[16];
 #pragma unroll
                     for (int u = 0; u < 16; ++u) {
                         const int k = wave + 4 * u;
-                        v[u] = (k < nk && lane < nvv) ? src[(long long)k * a.row] : 0.0f;
+                        v[u] = (k < nk && lane < nvv) ? src[(long long)key_pos(k) * a.row] : 0.0f;
                     }
 #pragma unroll
                     for (int u = 0; u < 16; ++u) Sl[(wave + 4 * u) * WSLAB + lane] = v[u];
@@ -265,7 +304,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
             for (int c = 0; c < WMAXC; ++c) r[m][c] = acc[m][i][c] * inv;
         }
         finish_row<M>(r, lane, a.dv, a.lambda, a.sub_norm, a.eps, a.out_scale, a.out + (long long)t * a.ldo + (long long)h * a.dv,
-                      a.gate ? a.gate + (long long)t * a.ldg + (long long)h * a.dv : nullptr);
+                      gate_of(a, t, h), a.head_gate ? 0 : 1);
     }
 }
 
@@ -306,7 +345,7 @@ __global__ __launch_bounds__(64) void window_attention_merge_kernel(const WinArg
         for (int c = 0; c < WMAXC; ++c) r[m][c] *= inv;
     }
     finish_row<M>(r, lane, a.dv, a.lambda, a.sub_norm, a.eps, a.out_scale, a.out + (long long)(row / a.H) * a.ldo + (long long)(row % a.H) * a.dv,
-                  a.gate ? a.gate + (long long)(row / a.H) * a.ldg + (long long)(row % a.H) * a.dv : nullptr);
+                  gate_of(a, row / a.H, row % a.H), a.head_gate ? 0 : 1);
 }
 
 // parts the key chunks of a row tile go round: only when few tiles face many chunks
@@ -319,10 +358,10 @@ static int window_splits(int T, int H, int G, int nkeys) {
     if (s > 64) s = 64;
     return s < 2 ? 1 : s;
 }
-static int window_keys(int pos0, int T, int window, int chunks) {
+static int window_keys(int pos0, int T, int window, int chunks, int keep) {
     const int all = pos0 + T;
     if (chunks && window > 0) return all - (pos0 / window) * window;     // from the start of the first token's chunk
-    return window > 0 && window + T - 1 < all ? window + T - 1 : all;
+    return window > 0 && (long long)window + T - 1 + keep < all ? window + T - 1 + keep : all;
 }
 
 }  // namespace ntk
@@ -344,17 +383,24 @@ int ntk_window_prepare_biased(float* cache, int row, float* q, int ldq, const fl
 }
 
 int ntk_window_prepare_ex(const ntk_window_prepare_desc* d, void* stream) {
-    if (!d || !d->cache || !d->q || !d->k || !d->v || !d->rot || (d->rot->dims > 0 && !d->rot->freq)) return NTK_E_NULL;
+    if (!d || !d->q || !d->rot || (d->rot->dims > 0 && !d->rot->freq)) return NTK_E_NULL;
+    if (d->k ? (!d->cache || !d->v) : (d->v || d->kb || d->vb || d->v_other || d->v_keep || d->k_norm)) return NTK_E_NULL;   // (without k: queries only)
     const ntk_rotary* rot = d->rot;
     if (d->temp_coef != 0.0f && !(d->temp_every > 0.0)) return NTK_E_SHAPE;
     if (d->T < 0 || d->H <= 0 || d->G <= 0 || d->H % d->G || d->maps < 1 || d->dn <= 0 || d->dv <= 0 || d->pos0 < 0) return NTK_E_SHAPE;
     if (rot->dims < 0 || (rot->dims & 1) || rot->dims > d->dn || (rot->layout != NTK_ROT_NEIGHBOURS && rot->layout != NTK_ROT_HALVES)) return NTK_E_SHAPE;
-    if (d->row < d->G * (d->maps * d->dn + d->dv) || d->ldq < d->H * d->maps * d->dn || d->ldk < d->G * d->maps * d->dn || d->ldv < d->G * d->dv) return NTK_E_SHAPE;
+    if (d->ldq < d->H * d->maps * d->dn) return NTK_E_SHAPE;
+    if (d->k && (d->row < d->G * (d->maps * d->dn + d->dv) || d->ldk < d->G * d->maps * d->dn || d->ldv < d->G * d->dv)) return NTK_E_SHAPE;
     if ((d->v_other && d->ld_other < d->G * d->dv) || (d->v_keep && d->ld_keep < d->G * d->dv)) return NTK_E_SHAPE;
     if (d->T == 0) return NTK_OK;
-    hipLaunchKernelGGL(window_prepare_kernel, dim3(d->T), dim3(256), (size_t)(rot->dims + 2) * sizeof(float), resolve_stream(stream), d->cache, d->row, d->q, d->ldq,
-                       d->k, d->ldk, d->v, d->ldv, d->H * d->maps, d->G * d->maps, d->dn, d->G * d->dv, rot->freq, rot->mag, rot->dims, d->pos0, d->qb, d->kb, d->vb,
-                       d->temp_coef, d->temp_every, rot->layout == NTK_ROT_HALVES ? 1 : 0, d->v_other, d->ld_other, d->v_blend, d->v_keep, d->ld_keep);
+    if (rot->dims > 16384) return NTK_E_SHAPE;     // (the angles' cos and sin sit in LDS)
+    const PrepareArgs a{d->cache, d->row, d->q, d->ldq, d->k, d->ldk, d->v, d->ldv, d->H * d->maps, d->G * d->maps, d->dn, d->G * d->dv, rot->freq, rot->mag, rot->dims,
+                        rot->layout == NTK_ROT_HALVES ? 1 : 0, d->pos0, d->qb, d->kb, d->vb, d->temp_coef, d->temp_every, d->v_other, d->ld_other, d->v_blend, d->v_keep,
+                        d->ld_keep, d->q_norm, d->k_norm, d->norm_eps};
+    const size_t lds = (size_t)(rot->dims + 2) * sizeof(float);
+    // a normed row is read twice, the second time behind a sum over the workgroup: few tokens (decoding) take workgroups of 1024
+    if ((d->q_norm || d->k_norm) && d->T <= 32) hipLaunchKernelGGL(window_prepare_kernel<1024>, dim3(d->T), dim3(1024), lds, resolve_stream(stream), a);
+    else hipLaunchKernelGGL(window_prepare_kernel<256>, dim3(d->T), dim3(256), lds, resolve_stream(stream), a);
     return last_launch_status();
 }
 
@@ -376,9 +422,11 @@ int ntk_window_attention(const ntk_window_attention_desc* d, void* stream) {
     a.pos0 = d->pos0; a.T = d->T; a.window = d->window; a.scale = d->scale; a.lambda = d->lambda; a.sub_norm = d->sub_norm; a.eps = d->eps; a.out_scale = d->out_scale;
     if ((d->mask_mode != NTK_MASK_SLIDING && d->mask_mode != NTK_MASK_CHUNKS) || d->softcap < 0.0f) return NTK_E_SHAPE;
     a.chunks = d->mask_mode == NTK_MASK_CHUNKS; a.softcap = d->softcap; a.sink = d->sink;
-    if (d->gate && d->ldg < d->H * d->dv) return NTK_E_SHAPE;
-    a.gate = d->gate; a.ldg = d->ldg;
-    a.splits = d->scratch ? window_splits(d->T, d->H, d->G, window_keys(d->pos0, d->T, d->window, a.chunks)) : 1;
+    if (d->gate && d->ldg < (d->head_gate ? d->H : d->H * d->dv)) return NTK_E_SHAPE;
+    a.gate = d->gate; a.ldg = d->ldg; a.head_gate = d->head_gate ? 1 : 0;
+    if (d->keep_first < 0 || (d->keep_first > 0 && a.chunks)) return NTK_E_SHAPE;
+    a.keep = d->keep_first; a.sinks = d->sinks;
+    a.splits = d->scratch ? window_splits(d->T, d->H, d->G, window_keys(d->pos0, d->T, d->window, a.chunks, a.keep)) : 1;
     a.scratch = d->scratch;
     a.rel = d->rel; a.bucket_of = d->bucket_of; a.n_dist = d->n_dist;
     if (a.rel && (!a.bucket_of || a.n_dist <= 0)) return NTK_E_NULL;

@@ -34,7 +34,8 @@ class WindowPrepareDesc(C.Structure):
     _fields_ = [("cache", C.c_void_p), ("row", C.c_int), ("q", C.c_void_p), ("ldq", C.c_int), ("k", C.c_void_p), ("ldk", C.c_int), ("v", C.c_void_p), ("ldv", C.c_int),
                 ("H", C.c_int), ("G", C.c_int), ("maps", C.c_int), ("dn", C.c_int), ("dv", C.c_int), ("rot", C.POINTER(Rotary)),
                 ("qb", C.c_void_p), ("kb", C.c_void_p), ("vb", C.c_void_p), ("temp_coef", C.c_float), ("temp_every", C.c_double),
-                ("v_other", C.c_void_p), ("ld_other", C.c_int), ("v_blend", C.c_float), ("v_keep", C.c_void_p), ("ld_keep", C.c_int), ("pos0", C.c_int), ("T", C.c_int)]
+                ("v_other", C.c_void_p), ("ld_other", C.c_int), ("v_blend", C.c_float), ("v_keep", C.c_void_p), ("ld_keep", C.c_int), ("pos0", C.c_int), ("T", C.c_int),
+                ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("norm_eps", C.c_float)]
 
 
 class WindowAttentionDesc(C.Structure):
@@ -42,7 +43,7 @@ class WindowAttentionDesc(C.Structure):
                 ("H", C.c_int), ("G", C.c_int), ("maps", C.c_int), ("dn", C.c_int), ("dv", C.c_int), ("pos0", C.c_int), ("T", C.c_int), ("window", C.c_int),
                 ("scale", C.c_float), ("lam", C.c_float), ("sub_norm", C.c_int), ("eps", C.c_float), ("out_scale", C.c_float), ("scratch", C.c_void_p),
                 ("rel", C.c_void_p), ("bucket_of", C.c_void_p), ("n_dist", C.c_int), ("mask_mode", C.c_int), ("softcap", C.c_float), ("sink", C.c_int),
-                ("gate", C.c_void_p), ("ldg", C.c_int)]
+                ("gate", C.c_void_p), ("ldg", C.c_int), ("head_gate", C.c_int), ("keep_first", C.c_int), ("sinks", C.c_void_p)]
 
 
 class GatedSeamDesc(C.Structure):
@@ -107,6 +108,8 @@ def _bind():
     L.ntk_lightning_attention_scratch.restype = C.c_size_t
     L.ntk_moe_route_ex.argtypes = [vp, vp, vp, vp, i, vp, vp, i, i, i, i, C.POINTER(RouteDesc), vp]
     L.ntk_glu.argtypes = [vp, vp, i, i, f, f, f, vp]
+    L.ntk_glu_rows.argtypes = [vp, i, vp, i, i, i, f, f, f, f, vp]
+    L.ntk_embed_bigram.argtypes = [vp, vp, vp, i, vp, i, i, i, i, i, f, i, ll, ll, vp]
     L.ntk_moe_sum.argtypes = [vp, vp, vp, vp, vp, vp, i, i, i, vp]
     L.ntk_dyt.argtypes = [vp, i, vp, i, vp, vp, f, i, i, vp]
     L.ntk_embed_positions.argtypes = [vp, vp, vp, vp, i, vp, i, i, i, i, i, vp, vp, f, vp]
@@ -388,9 +391,11 @@ def window_prepare_biased(q, k, v, H: int, G: int, dn: int, dv: int, pos0: int, 
 
 def window_attention(q: np.ndarray, cache: np.ndarray, H: int, G: int, maps: int, dn: int, dv: int, pos0: int, window: int, scale: float, lam: float = 0.0,
                      sub_norm: bool = False, eps: float = 1e-6, out_scale: float = 1.0, split: bool = True, rel: Optional[np.ndarray] = None,
-                     bucket_of: Optional[np.ndarray] = None, chunks: bool = False, softcap: float = 0.0, sink: bool = False, gate: Optional[np.ndarray] = None) -> np.ndarray:
+                     bucket_of: Optional[np.ndarray] = None, chunks: bool = False, softcap: float = 0.0, sink: bool = False, gate: Optional[np.ndarray] = None,
+                     keep_first: int = 0, sinks: Optional[np.ndarray] = None, head_gate: bool = False) -> np.ndarray:
     """q [T, H * maps * dn] (rotated), cache rows [G][maps][dn] keys | [G][dv] values; split: long key ranges of few rows may be cut into merged parts;
-    rel [buckets, H] with bucket_of [distances]: a bias by distance on the scaled score"""
+    rel [buckets, H] with bucket_of [distances]: a bias by distance on the scaled score; keep_first: positions that stay visible beside the window;
+    sinks [H]: the sink's score per head; gate [T, H * dv], or [T, H] with head_gate"""
     L = _bind()
     T, row = q.shape[0], G * (maps * dn + dv)
     qb, cb = _f(q), _f(cache)
@@ -402,9 +407,13 @@ def window_attention(q: np.ndarray, cache: np.ndarray, H: int, G: int, maps: int
         rb, bb = _f(rel), _i(bucket_of)
         d.rel, d.bucket_of, d.n_dist = rb.ptr, bb.ptr, len(bucket_of)
     d.mask_mode, d.softcap, d.sink = (MASK_CHUNKS if chunks else MASK_SLIDING), softcap, int(sink)
-    if gate is not None:        # [T, H * dv]: an elementwise sigmoid gate on the result
+    d.keep_first = keep_first
+    if sinks is not None:
+        kb = _f(sinks)
+        d.sinks = kb.ptr
+    if gate is not None:        # a sigmoid gate on the result
         gb = _f(gate)
-        d.gate, d.ldg = gb.ptr, gate.shape[1]
+        d.gate, d.ldg, d.head_gate = gb.ptr, gate.shape[1], int(head_gate)
     check(L.ntk_window_attention(C.byref(d), None), "ntk_window_attention")
     return out.numpy(np.float32, T * H * dv).reshape(T, H * dv)
 
@@ -566,27 +575,54 @@ def glu_cubic(gu: np.ndarray, ff: int, alpha: float, cubic: float, limit: float 
 
 
 def window_prepare_ex(q, k, v, H: int, G: int, dn: int, dv: int, pos0: int, freq=None, dims: int = 0, layout: int = ROT_NEIGHBOURS, v_other=None, v_blend: float = 0.0,
-                      keep: bool = False, cache: Optional[np.ndarray] = None, cache_rows: Optional[int] = None):
-    """one score map: rotation by `layout`, values blended with v_other [T, G * dv] on their way into the cache rows -> (cache, q, the values as they came if keep)"""
+                      keep: bool = False, cache: Optional[np.ndarray] = None, cache_rows: Optional[int] = None, mag: float = 1.0, q_norm=None, k_norm=None,
+                      norm_eps: float = 1e-6, qb=None, kb=None):
+    """one score map: (biases,) norms over the whole q / k with the weights q_norm / k_norm, rotation by `layout`, values blended with v_other [T, G * dv] on their
+    way into the cache rows -> (cache, q, the values as they came if keep); k None: queries only (the cache comes back as it was)"""
     L = _bind()
     T, row = q.shape[0], G * (dn + dv)
     n = cache_rows or (pos0 + T)
     cb = _f(cache) if cache is not None else DeviceBuffer.zeros(n * row * 4)
-    qd, kd, vd = _f(q), _f(k), _f(v)
+    opt = lambda x: _f(x) if x is not None else None
+    ptr = lambda b: b.ptr if b else None
+    qd, kd, vd, ob, qn, kn, qbias, kbias = _f(q), opt(k), opt(v), opt(v_other), opt(q_norm), opt(k_norm), opt(qb), opt(kb)
     fb = DeviceBuffer.from_numpy(np.ascontiguousarray(freq if freq is not None and len(freq) else [0.0], np.float64))
-    rot = Rotary(fb.ptr, 1.0, dims, layout)
-    ob = _f(v_other) if v_other is not None else None
-    kb = DeviceBuffer.zeros(T * G * dv * 4) if keep else None
+    rot = Rotary(fb.ptr, mag, dims, layout)
+    keep_b = DeviceBuffer.zeros(T * G * dv * 4) if keep else None
     d = WindowPrepareDesc()
-    d.cache, d.row, d.q, d.ldq, d.k, d.ldk, d.v, d.ldv = cb.ptr, row, qd.ptr, q.shape[1], kd.ptr, k.shape[1], vd.ptr, v.shape[1]
+    d.cache, d.row, d.q, d.ldq = cb.ptr, row, qd.ptr, q.shape[1]
+    if k is not None:
+        d.k, d.ldk, d.v, d.ldv = kd.ptr, k.shape[1], vd.ptr, v.shape[1]
     d.H, d.G, d.maps, d.dn, d.dv, d.rot, d.temp_every, d.pos0, d.T = H, G, 1, dn, dv, C.pointer(rot), 1.0, pos0, T
+    d.q_norm, d.k_norm, d.norm_eps, d.qb, d.kb = ptr(qn), ptr(kn), norm_eps, ptr(qbias), ptr(kbias)
     if ob:
         d.v_other, d.ld_other, d.v_blend = ob.ptr, G * dv, v_blend
-    if kb:
-        d.v_keep, d.ld_keep = kb.ptr, G * dv
+    if keep_b:
+        d.v_keep, d.ld_keep = keep_b.ptr, G * dv
     check(L.ntk_window_prepare_ex(C.byref(d), None), "ntk_window_prepare_ex")
     return (cb.numpy(np.float32, n * row).reshape(n, row), qd.numpy(np.float32, q.size).reshape(q.shape),
-            kb.numpy(np.float32, T * G * dv).reshape(T, G * dv) if kb else None)
+            keep_b.numpy(np.float32, T * G * dv).reshape(T, G * dv) if keep_b else None)
+
+
+def embed_bigram(table: np.ndarray, bigram: np.ndarray, tokens, prev: int, pos0: int, scale: float, mul_prev: int, mul_cur: int, dtype: str = "float32") -> np.ndarray:
+    """table [vocab, width], bigram [buckets + 1, width] -> [T, width]; prev: the token before tokens[0] (unused at pos0 0)"""
+    L = _bind()
+    T, (V, W) = len(tokens), table.shape
+    (tb, dt), (bb, _) = weight_buffer(table, dtype), weight_buffer(bigram, dtype)
+    ib = _i(tokens)
+    out = DeviceBuffer.zeros(T * W * 4)
+    check(L.ntk_embed_bigram(out.ptr, tb.ptr, bb.ptr, dt, ib.ptr, prev, pos0, T, V, W, scale, bigram.shape[0] - 1, mul_prev, mul_cur, None), "ntk_embed_bigram")
+    return out.numpy(np.float32, T * W).reshape(T, W)
+
+
+def glu_rows(gu: np.ndarray, ff: int, lda: int, limit: float = float("inf"), alpha: float = 1.0, cubic: float = 0.0, up_offset: float = 0.0) -> np.ndarray:
+    """the gated unit with output rows lda apart -> [rows, lda] (what lies behind the first ff columns stays zero)"""
+    L = _bind()
+    rows = gu.shape[0]
+    gb = _f(gu)
+    out = DeviceBuffer.zeros(rows * lda * 4)
+    check(L.ntk_glu_rows(out.ptr, lda, gb.ptr, gu.shape[1], rows, ff, limit, alpha, cubic, up_offset, None), "ntk_glu_rows")
+    return out.numpy(np.float32, rows * lda).reshape(rows, lda)
 
 
 def rms_seam(x: np.ndarray, w: Optional[np.ndarray], eps: float, add_y: Optional[np.ndarray] = None, add_w: Optional[np.ndarray] = None, mult: float = 1.0):
