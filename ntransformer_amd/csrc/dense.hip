@@ -31,7 +31,7 @@ struct DenseArgs {
     const void* W; long long wstride;
     const int* offsets;
     const int* rows; int row_div;
-    int T, N, K, accumulate, G, vec;
+    int T, N, K, accumulate, G, vec, xvec;   // vec: weight rows 16-byte aligned, K % 8 == 0; xvec: activation rows (and norm_w) 16-byte aligned, K % 4 == 0
     int glu_ff; float glu_limit, glu_alpha, glu_up_offset, glu_cubic;   // few-row form only: outputs f < glu_ff = gated unit of rows f (gate) and glu_ff + f (up)
     const float* norm_w; float norm_eps, norm_offset;   // few-row form only: the activation row is RMS-normed with weight (offset + norm_w) first
 };
@@ -143,19 +143,29 @@ __global__ __launch_bounds__(256) void dense_mfma_kernel(const DenseArgs a) {
 #pragma unroll
             for (int j = 0; j < NJ; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af[i], bfr[j], acc[i][j], 0, 0, 0);
     }
-    // accumulator lane map: row 4 * (lane / 16) + r, column lane % 16
+    // accumulator lane map: row 4 * (lane / 16) + r, column lane % 16.  What a sum is added onto is requested for a whole strip of tiles before the first store.
 #pragma unroll
-    for (int i = 0; i < MI; ++i)
+    for (int i = 0; i < MI; ++i) {
+        const int row = row_base + wm * (TM / 2) + i * 16 + (lane >> 4) * 4;
+        float* y = a.Y + (long long)row * a.ldy + n_base + wn * (TN / 2) + (lane & 15);
+        const int n_left = a.N - (n_base + wn * (TN / 2) + (lane & 15));
+        if (a.accumulate) {                                  // (uniform over the launch)
+            float old[NJ][4];
+#pragma unroll
+            for (int j = 0; j < NJ; ++j)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) old[j][r] = row + r < r1 && j * 16 < n_left ? y[(long long)r * a.ldy + j * 16] : 0.0f;
+#pragma unroll
+            for (int j = 0; j < NJ; ++j)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) acc[i][j][r] += old[j][r];
+        }
 #pragma unroll
         for (int j = 0; j < NJ; ++j)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int row = row_base + wm * (TM / 2) + i * 16 + (lane >> 4) * 4 + r, col = n_base + wn * (TN / 2) + j * 16 + (lane & 15);
-                if (row < r1 && col < a.N) {
-                    float* y = a.Y + (long long)row * a.ldy + col;
-                    *y = a.accumulate ? *y + acc[i][j][r] : acc[i][j][r];
-                }
-            }
+            for (int r = 0; r < 4; ++r)
+                if (row + r < r1 && j * 16 < n_left) y[(long long)r * a.ldy + j * 16] = acc[i][j][r];
+    }
 }
 
 // ---------------------------------------------------------------------------------------------------------------- float32, vector FMA
@@ -229,53 +239,96 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
         while (r >= a.offsets[g + 1]) ++g;
     }
     const float* xrow = a.X + (long long)(a.rows ? a.rows[r] / a.row_div : r) * a.ldx;
-    float ss = 0.0f;
-    for (int k = threadIdx.x; k < a.K; k += 256) { const float v = xrow[k]; xs[k] = v; ss = fmaf(v, v, ss); }
-    if (a.norm_w) {                                         // (uniform over the launch)
-        __shared__ float red[16];
-        ss = block_sum(ss, red);
-        const float inv = 1.0f / sqrtf(ss / (float)a.K + a.norm_eps);
-        for (int k = threadIdx.x; k < a.K; k += 256) xs[k] = xs[k] * inv * (a.norm_offset + a.norm_w[k]);   // (each thread rewrites what it wrote)
-    }
-    __syncthreads();
     const WT* W = (const WT*)a.W + (long long)g * a.wstride;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     // GLU: the wave's RW rows are RW / 2 (gate, up) pairs of RW / 2 consecutive outputs
     constexpr int OUT = GLU ? RW / 2 : RW;
     const int n_out = GLU ? a.glu_ff : a.N;
     const int n0 = (blockIdx.x * 4 + wave) * OUT;
-    if (n0 >= n_out) return;                                // uniform per wave
     const WT* w[RW];
 #pragma unroll
     for (int i = 0; i < RW; ++i) {                          // rows past the end re-read the last one and are not stored
         const int row = GLU ? (i < OUT ? min(n0 + i, n_out - 1) : a.glu_ff + min(n0 + i - OUT, n_out - 1)) : min(n0 + i, n_out - 1);
         w[i] = W + (long long)row * a.K;
     }
+    constexpr int NV = sizeof(WT) == 2 ? 1 : 2;             // 16-byte pieces of eight weights
+    auto weights = [&](uintx4_t (&u)[RW][NV], int k) {
+#pragma unroll
+        for (int i = 0; i < RW; ++i)
+#pragma unroll
+            for (int p = 0; p < NV; ++p) u[i][p] = __builtin_nontemporal_load(reinterpret_cast<const uintx4_t*>(w[i] + k) + p);
+    };
+    float ss = 0.0f;
+    uintx4_t first[RW][NV];
+    if (a.xvec) {
+        // the row's first 4096 entries stay in registers up to the norm; they, their norm weights and the wave's first weights are requested together
+        constexpr int XV = 4;
+        float4 xv[XV], nv[XV];
+#pragma unroll
+        for (int u = 0; u < XV; ++u) {
+            const int k = 4 * (tid + 256 * u);
+            xv[u] = k < a.K ? *reinterpret_cast<const float4*>(xrow + k) : float4{0.0f, 0.0f, 0.0f, 0.0f};
+            nv[u] = a.norm_w && k < a.K ? *reinterpret_cast<const float4*>(a.norm_w + k) : float4{0.0f, 0.0f, 0.0f, 0.0f};
+        }
+        if (a.vec && lane * 8 < a.K) weights(first, lane * 8);
+        for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256) *reinterpret_cast<float4*>(xs + k) = *reinterpret_cast<const float4*>(xrow + k);
+        float inv = 1.0f;
+        if (a.norm_w) {                                     // (uniform over the launch)
+            __shared__ float red[16];
+#pragma unroll
+            for (int u = 0; u < XV; ++u) { ss = fmaf(xv[u].x, xv[u].x, ss); ss = fmaf(xv[u].y, xv[u].y, ss); ss = fmaf(xv[u].z, xv[u].z, ss); ss = fmaf(xv[u].w, xv[u].w, ss); }
+            for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) ss = fmaf(xs[k + j], xs[k + j], ss);
+            inv = 1.0f / sqrtf(block_sum(ss, red) / (float)a.K + a.norm_eps);
+            for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) xs[k + j] = xs[k + j] * inv * (a.norm_offset + a.norm_w[k + j]);   // (each thread rewrites what it wrote)
+        }
+#pragma unroll
+        for (int u = 0; u < XV; ++u) {
+            const int k = 4 * (tid + 256 * u);
+            if (k >= a.K) continue;
+            float4 v = xv[u];
+            if (a.norm_w) { v.x = v.x * inv * (a.norm_offset + nv[u].x); v.y = v.y * inv * (a.norm_offset + nv[u].y); v.z = v.z * inv * (a.norm_offset + nv[u].z); v.w = v.w * inv * (a.norm_offset + nv[u].w); }
+            *reinterpret_cast<float4*>(xs + k) = v;
+        }
+    } else {
+        if (a.vec && lane * 8 < a.K) weights(first, lane * 8);
+        for (int k = tid; k < a.K; k += 256) { const float v = xrow[k]; xs[k] = v; ss = fmaf(v, v, ss); }
+        if (a.norm_w) {
+            __shared__ float red[16];
+            ss = block_sum(ss, red);
+            const float inv = 1.0f / sqrtf(ss / (float)a.K + a.norm_eps);
+            for (int k = tid; k < a.K; k += 256) xs[k] = xs[k] * inv * (a.norm_offset + a.norm_w[k]);   // (each thread rewrites what it wrote)
+        }
+    }
+    __syncthreads();
+    if (n0 >= n_out) return;                                // uniform per wave
     float s[RW];
 #pragma unroll
     for (int i = 0; i < RW; ++i) s[i] = 0.0f;
     if (a.vec) {
-#pragma unroll 2
+        uintx4_t cur[RW][NV], next[RW][NV];
+#pragma unroll
+        for (int i = 0; i < RW; ++i)
+#pragma unroll
+            for (int p = 0; p < NV; ++p) cur[i][p] = first[i][p];
         for (int k = lane * 8; k < a.K; k += 64 * 8) {
+            if (k + 64 * 8 < a.K) weights(next, k + 64 * 8);        // the next pass's weights behind this pass's sums
             float wv[RW][8];
-            if constexpr (sizeof(WT) == 2) {
-                uintx4_t u[RW];
 #pragma unroll
-                for (int i = 0; i < RW; ++i) u[i] = __builtin_nontemporal_load(reinterpret_cast<const uintx4_t*>(w[i] + k));
-#pragma unroll
-                for (int i = 0; i < RW; ++i) {
-                    const uint32_t uu[4] = {u[i].x, u[i].y, u[i].z, u[i].w};
+            for (int i = 0; i < RW; ++i) {
+                if constexpr (sizeof(WT) == 2) {
+                    const uint32_t uu[4] = {cur[i][0].x, cur[i][0].y, cur[i][0].z, cur[i][0].w};
 #pragma unroll
                     for (int j = 0; j < 4; ++j) { wv[i][2 * j] = __uint_as_float(uu[j] << 16); wv[i][2 * j + 1] = __uint_as_float(uu[j] & 0xffff0000u); }
-                }
-            } else {
-                float4 u0[RW], u1[RW];
+                } else {
 #pragma unroll
-                for (int i = 0; i < RW; ++i) { u0[i] = *reinterpret_cast<const float4*>(w[i] + k); u1[i] = *reinterpret_cast<const float4*>(w[i] + k + 4); }
-#pragma unroll
-                for (int i = 0; i < RW; ++i) {
-                    wv[i][0] = u0[i].x; wv[i][1] = u0[i].y; wv[i][2] = u0[i].z; wv[i][3] = u0[i].w;
-                    wv[i][4] = u1[i].x; wv[i][5] = u1[i].y; wv[i][6] = u1[i].z; wv[i][7] = u1[i].w;
+                    for (int p = 0; p < 2; ++p) {
+                        wv[i][4 * p] = __uint_as_float(cur[i][p].x); wv[i][4 * p + 1] = __uint_as_float(cur[i][p].y);
+                        wv[i][4 * p + 2] = __uint_as_float(cur[i][p].z); wv[i][4 * p + 3] = __uint_as_float(cur[i][p].w);
+                    }
                 }
             }
             const float4 x0 = *reinterpret_cast<const float4*>(xs + k), x1 = *reinterpret_cast<const float4*>(xs + k + 4);
@@ -284,6 +337,10 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
             for (int i = 0; i < RW; ++i)
 #pragma unroll
                 for (int j = 0; j < 8; ++j) s[i] = fmaf(wv[i][j], xv[j], s[i]);
+#pragma unroll
+            for (int i = 0; i < RW; ++i)
+#pragma unroll
+                for (int p = 0; p < NV; ++p) cur[i][p] = next[i][p];
         }
     } else {
         for (int k = lane; k < a.K; k += 64) {
@@ -351,13 +408,14 @@ int ntk_dense(const ntk_dense_desc* d, void* stream) {
     if (d->norm_w && d->T > kGemvRows) return NTK_E_SHAPE;
     if (d->T == 0) return NTK_OK;
     const int G = d->offsets ? d->G : 1;
-    DenseArgs a{d->Y, d->ldy, d->X, d->ldx, d->W, d->wstride, d->offsets, d->rows, d->rows ? d->row_div : 1, d->T, d->N, d->K, d->accumulate, G, 0, 0, 0.0f, 0.0f, 0.0f, 0.0f, nullptr, 0.0f, 0.0f};
+    DenseArgs a{d->Y, d->ldy, d->X, d->ldx, d->W, d->wstride, d->offsets, d->rows, d->rows ? d->row_div : 1, d->T, d->N, d->K, d->accumulate, G, 0, 0, 0, 0.0f, 0.0f, 0.0f, 0.0f, nullptr, 0.0f, 0.0f};
     hipStream_t s = resolve_stream(stream);
     if (d->T <= kGemvRows) {
         if ((size_t)d->K * 4 > 160 * 1024 - 1024) return NTK_E_SHAPE;
         a.glu_ff = d->glu_ff; a.glu_limit = d->glu_limit; a.glu_alpha = d->glu_alpha; a.glu_up_offset = d->glu_up_offset; a.glu_cubic = d->glu_cubic;
         a.norm_w = d->norm_w; a.norm_eps = d->norm_eps; a.norm_offset = d->norm_offset;
         a.vec = (d->K % 8 == 0) && !((uintptr_t)d->W & 15) && !((d->wstride * (d->wdtype == NTK_DT_BF16 ? 2 : 4)) & 15);
+        a.xvec = (d->K % 4 == 0) && (d->ldx % 4 == 0) && !((uintptr_t)d->X & 15) && !((uintptr_t)d->norm_w & 15);
         if (d->wdtype == NTK_DT_BF16) launch_gemv<uint16_t>(a, d->T, s);
         else launch_gemv<float>(a, d->T, s);
         return last_launch_status();

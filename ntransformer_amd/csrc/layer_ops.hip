@@ -30,17 +30,16 @@ template <typename TT> __device__ __forceinline__ float table_value(const TT* ro
 template <typename TT>
 __global__ __launch_bounds__(256) void embed_bigram_kernel(float* out, const TT* table, const TT* bigram, const int* tokens, int prev, int pos0, int vocab, int width,
                                                            float scale, int buckets, long long mul_prev, long long mul_cur) {
-    const int t = blockIdx.x, tok = tokens[t];
-    float* o = out + (long long)t * width;
+    const int t = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x, tok = tokens[t];
+    if (i >= width) return;
     const bool ok = tok >= 0 && tok < vocab;
     long long r = buckets;                                   // a sequence's first token
     if (pos0 + t > 0) {
         r = ((long long)(t > 0 ? tokens[t - 1] : prev) * mul_prev + (long long)tok * mul_cur) % buckets;
         if (r < 0) r += buckets;
     }
-    const TT* row = table + (long long)(ok ? tok : 0) * width;
-    const TT* two = bigram + r * width;
-    for (int i = threadIdx.x; i < width; i += 256) o[i] = fmaf(ok ? table_value(row, i) : 0.0f, scale, table_value(two, i));
+    const float e = table_value(table + (long long)(ok ? tok : 0) * width, i), b = table_value(bigram + r * width, i);
+    out[(long long)t * width + i] = fmaf(ok ? e : 0.0f, scale, b);
 }
 
 __global__ __launch_bounds__(256) void rmsnorm_offset_kernel(float* y1, const float* w1, float* y2, const float* w2, int ldy, const float* x, int ldx, int n,
@@ -241,11 +240,12 @@ int ntk_embed_bigram(float* out, const void* table, const void* bigram, int tdty
     if (tdtype != NTK_DT_BF16 && tdtype != NTK_DT_F32) return NTK_E_DTYPE;
     if (T < 0 || vocab <= 0 || width <= 0 || pos0 < 0 || buckets <= 0) return NTK_E_SHAPE;
     if (T == 0) return NTK_OK;
+    const dim3 grid((width + 255) / 256, T);
     if (tdtype == NTK_DT_BF16)
-        hipLaunchKernelGGL(embed_bigram_kernel<uint16_t>, dim3(T), dim3(256), 0, resolve_stream(stream), out, (const uint16_t*)table, (const uint16_t*)bigram, tokens, prev,
+        hipLaunchKernelGGL(embed_bigram_kernel<uint16_t>, grid, dim3(256), 0, resolve_stream(stream), out, (const uint16_t*)table, (const uint16_t*)bigram, tokens, prev,
                            pos0, vocab, width, scale, buckets, mul_prev, mul_cur);
     else
-        hipLaunchKernelGGL(embed_bigram_kernel<float>, dim3(T), dim3(256), 0, resolve_stream(stream), out, (const float*)table, (const float*)bigram, tokens, prev, pos0,
+        hipLaunchKernelGGL(embed_bigram_kernel<float>, grid, dim3(256), 0, resolve_stream(stream), out, (const float*)table, (const float*)bigram, tokens, prev, pos0,
                            vocab, width, scale, buckets, mul_prev, mul_cur);
     return last_launch_status();
 }

@@ -179,17 +179,18 @@ def tubazen_shapes(cfg: dict, buckets: int = 32, rank: int = 64) -> Dict[str, Tu
     return s
 
 
-def fifotar_config(preset: str, layers: int = 4, mlp_everywhere: bool = True) -> dict:
+def fifotar_config(preset: str, layers: int = 4, mlp_everywhere: bool = True, attention_only: bool = False) -> dict:
     """the scaled family at the preset's width, heads and vocabulary: chunked attention (four query heads per key/value head, chunks of the preset's window,
     capped scores, blended values), the per-head delta rule (two value heads per key head, keys and values of the preset's sizes, four taps) and latent
-    attention (the preset's ranks) in the order attention, delta, latent, delta; the clipped gated feed-forward with the bytes of the gated family's"""
+    attention (the preset's ranks) in the order attention, delta, latent, delta (attention_only: nothing but the first); the clipped gated feed-forward with the
+    bytes of the gated family's"""
     p = PRESETS[preset]
     H, dn, dv = p["heads"], p["dim"], p["vdim"]
     ff = (p["top"] * p["ff"] + p["shared_ff"]) * 2 // 3
     ff -= ff % 64
     ls = []
     for k in range(layers):
-        if k % 4 == 0:
+        if k % 4 == 0 or attention_only:
             mx = {"heads": H, "kv_heads": max(H // 4, 1), "dim": dn, "vdim": dv, "scale": 1.0 / math.sqrt(dn), "softcap": 40.0, "mask": {"size": p["window"]}, "v_mix": True}
             t = "attention"
         elif k % 4 == 2:
@@ -235,9 +236,47 @@ def fifotar_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
     return s
 
 
+def zalazen_config(preset: str, layers: int = 4) -> dict:
+    """the dense parallel family at the preset's width, heads and vocabulary: sliding-window attention (four query heads per key/value head, the preset's window and
+    four kept first positions, every dimension rotated), every second layer reading the keys and values of the one before it, and the dense gated feed-forward of
+    fifotar_config"""
+    p = PRESETS[preset]
+    H, dn, dv = p["heads"], p["dim"], p["vdim"]
+    ff = (p["top"] * p["ff"] + p["shared_ff"]) * 2 // 3
+    ff -= ff % 64
+    ls = []
+    for k in range(layers):
+        mx = {"heads": H, "kv_heads": max(H // 4, 1), "dim": dn, "vdim": dv, "scale": 1.0 / math.sqrt(dn), "mask": {"size": p["window"], "keep_first": 4},
+              "rot": {"base": 500000.0, "dims": dn, "scaling": {"factor": 8.0, "original": 4096, "fast": 16.0, "slow": 2.0}}}
+        if k % 2:
+            mx["kv_from"] = k - 1
+        ls.append({"type": "attention", "mixer": mx, "mlp": {"kind": "dense", "ff": max(ff, 64)}})
+    return {"architecture": "Zalazen", "layers": ls, "norm": {"eps": 1e-5}, "vocab": p["vocab"], "width": p["width"],
+            "embedding": {"scale": math.sqrt(p["width"]), "bigram": {"buckets": p["vocab"] // 2 - 1, "mul_prev": 1009, "mul_cur": 31}}}
+
+
+def zalazen_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
+    W, V = cfg["width"], cfg["vocab"]
+    s: Dict[str, Tuple[int, ...]] = {"embed": (V, W), "head": (V, W), "final.norm": (W,)}
+    if cfg["embedding"].get("bigram"):
+        s["bigram"] = (cfg["embedding"]["bigram"]["buckets"] + 1, W)
+    for i, L in enumerate(cfg["layers"]):
+        p, mx, ml = "l%d." % i, L["mixer"], L.get("mlp")
+        H, G, dn, dv, q = mx["heads"], mx.get("kv_heads", mx["heads"]), mx["dim"], mx["vdim"], p + "mix."
+        s[p + "norm1"] = (W,)
+        s[q + "q"], s[q + "q.norm"], s[q + "g"], s[q + "sink"], s[q + "o"] = (H * dn, W), (H * dn,), (H, W), (H,), (W, H * dv)
+        if mx.get("kv_from") is None:
+            s[q + "k"], s[q + "k.norm"], s[q + "v"] = (G * dn, W), (G * dn,), (G * dv, W)
+        if ml:
+            s[p + "norm2"] = (W,)
+            s[p + "mlp.gate"], s[p + "mlp.up"], s[p + "mlp.down"] = (ml["ff"], W), (ml["ff"], W), (W, ml["ff"])
+    return s
+
+
 def shapes_of(cfg: dict) -> Dict[str, Tuple[int, ...]]:
     arch = cfg.get("architecture")
     return (nizorax_shapes(cfg) if arch == "Nizorax" else tubazen_shapes(cfg) if arch == "Tubazen" else fifotar_shapes(cfg) if arch == "Fifotar" else
+            zalazen_shapes(cfg) if arch == "Zalazen" else
             fabolorn_shapes(cfg))
 
 
@@ -278,7 +317,7 @@ def write_folder(folder: str, cfg: dict, seed: int = 20260925) -> int:
                     around_one = name.rsplit(".", 1)[-1] in ("norm", "norm1", "norm2")
                 if cfg.get("architecture") == "Nizorax":     # layer-norm weights around one, biases / lambda vectors / activation numbers small
                     around_one = name.rsplit(".", 1)[-1] in ("norm", "norm1", "norm2", "norm1b", "norm2b")
-                if cfg.get("architecture") == "Fifotar":     # every norm weight is stored plain; decay rates and biases small
+                if cfg.get("architecture") in ("Fifotar", "Zalazen"):     # every norm weight is stored plain; decay rates and biases small
                     around_one = "norm" in name.rsplit(".", 1)[-1]
                 vals = 0.1 * pool[:n] + (1.0 if around_one else 0.0)
                 f.write(_bf16(vals).tobytes())
