@@ -226,8 +226,9 @@ __global__ __launch_bounds__(256) void dense_fma_kernel(const DenseArgs a) {
 
 // ---------------------------------------------------------------------------------------------------------------- few rows: waves stream weight rows
 // One workgroup per (group of 4 * RW outputs, activation row): the activation row sits in LDS, each wave owns RW consecutive weight rows and walks
-// them together -- per step a lane requests 16 bytes of each of its RW rows before it uses any (RW loads in flight per lane), reads its 8 activations
-// once and feeds RW sums; one DPP reduction per row at the end.  RW is picked so that the launch still has a few workgroups per CU.
+// them together -- per step a lane requests the NEXT 16 bytes of each of its RW rows, then reads its 8 activations once and feeds RW sums from the bytes that
+// have arrived; one DPP reduction per row at the end.  The first weights are requested together with the activation row and the weights of its norm, so they
+// travel behind the norm's sum over the workgroup.  RW is picked so that the launch still has a few workgroups per CU.
 constexpr int kGemvRows = 8;       // up to this many rows take this form
 template <typename WT, int RW, bool GLU>
 __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
