@@ -60,11 +60,11 @@ def parse():
     ap.add_argument("--cpu-tokens", type=int, default=128, help="-n of the reference CLI run that is the CPU baseline (BASELINE config 1: 128)")
     ap.add_argument("--no-also", action="store_true", help="skip the other BASELINE configurations (8B Q4_K_M, 70B Q4_K_M, 70B Q6_K, 8B Q8_0 behind 3900- and 32768-token prompts)")
     ap.add_argument("--no-pmc-note", action="store_true")
-    ap.add_argument("--family", default="", choices=["", "fabolorn", "nizorax", "tubazen", "fifotar", "zalazen"],
+    ap.add_argument("--family", default="", choices=["", "fabolorn", "nizorax", "tubazen", "fifotar", "zalazen", "gibevik"],
                     help="instead of the default workload: prompt and decode throughput of a layer-list family on synthetic real-sized layers; beside it, fabolorn: the "
                          "Llama path at equal width / heads / active feed-forward width (F16 and Q8_0), nizorax: the fabolorn family at the same preset, tubazen: the nizorax "
                          "family at the same preset with the dense feed-forward in every layer, fifotar: the tubazen family at the same preset and number of layers, zalazen: the fifotar family's attention layers "
-                         "at the same preset and number of layers; "
+                         "at the same preset and number of layers, gibevik: the fifotar family with latent and attention layers and the fabolorn family; "
                          "one JSON line of its own")
     ap.add_argument("--family-size", default="lite", choices=["tiny", "lite", "mid"])
     ap.add_argument("--family-no-compare", action="store_true", help="skip the runs beside the family (a profile of the family's kernels alone)")
@@ -427,7 +427,7 @@ def time_folder(args, cfg, prompt, ctx):
 
 
 def run_family(args):
-    """--family fabolorn | nizorax | tubazen | fifotar | zalazen: a synthetic model folder of `--family-layers` real-sized layers (ntransformer_amd/synth_folder.py), a prompt pass of
+    """--family fabolorn | nizorax | tubazen | fifotar | zalazen | gibevik: a synthetic model folder of `--family-layers` real-sized layers (ntransformer_amd/synth_folder.py), a prompt pass of
     --prompt-bench tokens (second of two runs) and --steps decoded tokens behind it through the slot cache.  Beside it, unless --family-no-compare:
     fabolorn -- the Llama path with the same width, heads (head size 128), layers, vocabulary and ACTIVE feed-forward width (top x ff + shared ff) as
     F16 and as Q8_0, same prompt and decode; nizorax -- the Fabolorn family (the closest model: same layer stack, slots and products) at the same preset;
@@ -435,7 +435,9 @@ def run_family(args):
     (equal feed-forward bytes: three matrices here, two there); fifotar -- the Tubazen family (the closest model: attention beside a delta-rule recurrence, a
     gated dense feed-forward of the same three matrices) at the same preset and number of layers (its layers go attention, delta, latent attention, delta:
     --family-layers 4 shows every mixer); zalazen -- the Fifotar family with nothing but attention layers (the closest model: the same attention kernels over the same
-    number of keys, heads and sizes, a gated dense feed-forward of the same bytes) at the same preset and number of layers."""
+    number of keys, heads and sizes, a gated dense feed-forward of the same bytes) at the same preset and number of layers; gibevik -- the Fifotar family with latent, latent, attention,
+    attention layers (the closest model for everything but the experts: the same latent and grouped-query kernels, sizes and feed-forward bytes) and the Fabolorn family
+    (the closest mixture of experts) at the same preset and number of layers (--family-layers 4 shows every mixer)."""
     import numpy as np
     from ntransformer_amd import _lib, synth_folder
     from ntransformer_amd import engine as E
@@ -446,7 +448,12 @@ def run_family(args):
     rng = np.random.Generator(np.random.Philox(key=[20260925, 7]))
     prompt = [int(t) for t in rng.integers(0, p["vocab"], T)]
     out = {}
-    if args.family == "zalazen":
+    if args.family == "gibevik":
+        out["gibevik"] = time_folder(args, synth_folder.gibevik_config(args.family_size, args.family_layers), prompt, ctx)
+        if not args.family_no_compare:
+            out["fifotar"] = time_folder(args, synth_folder.fifotar_config(args.family_size, args.family_layers, order=("latent_attention", "latent_attention", "attention", "attention")), prompt, ctx)
+            out["fabolorn"] = time_folder(args, synth_folder.fabolorn_config(args.family_size, args.family_layers), prompt, ctx)
+    elif args.family == "zalazen":
         out["zalazen"] = time_folder(args, synth_folder.zalazen_config(args.family_size, args.family_layers), prompt, ctx)
         if not args.family_no_compare:
             out["fifotar"] = time_folder(args, synth_folder.fifotar_config(args.family_size, args.family_layers, attention_only=True), prompt, ctx)

@@ -46,7 +46,16 @@ typedef struct ntk_dense_desc {
     /* a cubic term inside the gate's sigmoid: act(g') = g' * sigmoid(glu_alpha * (g' + glu_cubic * g'^3)).  0: none.  alpha = 2 sqrt(2 / pi) and
      * cubic = 0.044715 give the tanh form of gelu, 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))), since 0.5 (1 + tanh y) = sigmoid(2 y) */
     float glu_cubic;
+    /* an activation on the product itself, in every form (not with accumulate or glu_ff): NTK_ACT_RELU2: Y = max(y, 0)^2 */
+    int act;
+    /* add_y != NULL (only with T <= ntk_dense_few_rows(), no rows / offsets): the activation row is X[r] + add_mult * add_y[r] / sqrt(mean(add_y[r]^2) + add_eps) * add_w
+     * (add_w F32 [K]; norm_w then norms that sum) and x_out receives it (rows ldxo floats apart; must not overlap X or add_y) -- ntk_rms_seam and the product in one
+     * launch: what a sublayer still owes to the stream joins it on the way into the next sublayer's first product */
+    const float* add_y; int ld_add; const float* add_w; float add_eps, add_mult;
+    float* x_out; int ldxo;
 } ntk_dense_desc;
+#define NTK_ACT_NONE 0
+#define NTK_ACT_RELU2 1
 int ntk_dense_few_rows(void);   /* up to this many rows a product takes the row-streaming form */
 int ntk_dense(const ntk_dense_desc* d, void* stream);
 /* the plain case: Y[T][N] = X[T][K] . W[N][K]^T */
@@ -75,6 +84,9 @@ int ntk_embed_dense_scaled(float* out, const void* table, int tdtype, const int*
  * in the table's dtype.  prev is the token before tokens[0] (unused when pos0 == 0). */
 int ntk_embed_bigram(float* out, const void* table, const void* bigram, int tdtype, const int* tokens, int prev, int pos0, int T, int vocab, int width, float scale,
                      int buckets, long long mul_prev, long long mul_cur, void* stream);
+/* out[t][:] = table[tokens[t]][:] * scale + u(pos0 + t), u(p)_{2i} = sin(p * freq[i]), u(p)_{2i+1} = cos(p * freq[i]) -- a sinusoidal position vector; freq device
+ * F64 [(width + 1) / 2], angles formed in double */
+int ntk_embed_sinusoid(float* out, const void* table, int tdtype, const int* tokens, int T, int vocab, int width, float scale, const double* freq, int pos0, void* stream);
 /* x[i] *= s */
 int ntk_scale(float* x, long long n, float s, void* stream);
 /* Layer norm with weight and bias: y[t][:] (+)= (x[t] - mean) / sqrt(var + eps) * w + b, var = mean of the squared deviations (two passes).
@@ -160,7 +172,7 @@ typedef struct ntk_rotary {       /* angle of pair i at position p: p * freq[i];
 #define NTK_ROT_HALVES 1
 /* For T tokens at positions pos0 ...: kv [T][ldkv] = [kv_rank raw latent | rot_dim raw key part] -> cache rows pos0 .. pos0+T-1:
  * latent / rms * norm_w, key part rotated (its first rot->dims entries, paired by rot->layout; the rest copied).  q [T][H][qd], ldq floats between tokens: the rot_dim entries at the
- * end of every head rotated in place the same way. */
+ * end of every head rotated in place the same way.  rot == NULL: nothing is rotated (the key part is copied, q is left alone). */
 int ntk_latent_prepare(float* cache, int row, const float* kv, int ldkv, const float* norm_w, float eps, int kv_rank, int rot_dim, float* q, int ldq, int H, int qd,
                        const ntk_rotary* rot, int pos0, int T, void* stream);
 /* Softmax attention of query rows over cached positions.  Two forms of one kernel:
@@ -176,6 +188,10 @@ int ntk_latent_attention(float* out, int ldo, const float* q, int ldq, const flo
                          void* stream);
 /* fold the unrotated query part through the key up-projection: qf[t][h][0..R) = sum_d q[t][h][d] * W_uk[h*dn + d][0..R), and copy the rotated part behind it
  * (qf [T][H][R+dr]; q rows ldq floats apart); W_uk NTK_DT_BF16 / F32 [H*dn][R] */
+/* ... and, beside it in the same launch, the latents of these tokens into the cache rows: kv [T][ldkv] raw latents -> kv / rms * norm_w (ntk_latent_prepare without a
+ * rotated part, dr == 0 only: then the fold reads nothing that it writes) */
+int ntk_latent_fold_query_prepare(float* qf, const float* q, int ldq, const void* w_uk, int wdtype, int T, int H, int dn, int R, float* cache, int row, const float* kv,
+                                  int ldkv, const float* norm_w, float eps, int pos0, void* stream);
 int ntk_latent_fold_query(float* qf, const float* q, int ldq, const void* w_uk, int wdtype, int T, int H, int dn, int dr, int R, void* stream);
 /* out[t][h*dv + v] = sum_r W_uv[h*dv + v][r] * lat[t][h][r]  (the value up-projection applied after the weighted sum), times sigmoid(gate[t][h*dv+v]) if gate */
 int ntk_latent_unfold_value(float* out, int ldo, const float* lat, const void* w_uv, int wdtype, const float* gate, int ldg, int T, int H, int dv, int R,
@@ -215,6 +231,9 @@ typedef struct ntk_window_prepare_desc {
      * sqrt(mean(x^2) + norm_eps), the mean over ALL heads at once, times the weight, ahead of the rotation.
      * k == NULL (then v, cache and everything of theirs too): only q is treated -- a layer that reads the cache rows of another one. */
     const float* q_norm; const float* k_norm; float norm_eps;
+    /* head_norm != 0: the norm runs over every head's dn entries (per map) on its own, with ONE weight vector [dn] for all heads (q_norm [dn] / k_norm [dn]), and the
+     * query temperature multiplies the NORMED query.  v may be the same memory as k: values that are the keys as they were projected. */
+    int head_norm;
 } ntk_window_prepare_desc;
 int ntk_window_prepare_ex(const ntk_window_prepare_desc* d, void* stream);
 /* a_m = softmax_j(scale * q_m . k_m[j]) V over the visible j (j <= p, and p - j < window if window > 0), per map m.
@@ -245,6 +264,8 @@ typedef struct ntk_window_attention_desc {
      * sinks != NULL (device F32 [H]): the sink's score is sinks[h] (unscaled, once per head) instead of 0; `sink` need not be set. */
     int head_gate, keep_first;
     const float* sinks;
+    /* slopes != NULL (device F32 [H]): slopes[h] * (p - j) is taken off the scaled score: a bias that falls with the distance, each head at its own rate */
+    const float* slopes;
 } ntk_window_attention_desc;
 #define NTK_MASK_SLIDING 0
 #define NTK_MASK_CHUNKS 1
@@ -317,15 +338,37 @@ int ntk_moe_route(int* ids, float* wts, float* sgate, const float* h, int ldh, c
                   void* stream);
 /* The general router.  score 0: s = softmax(z), 1: s = sigmoid(z).  groups > 1: the experts form `groups` equal groups of neighbours, a group's
  * score is the sum of its `group_top` largest s, and only experts of the `keep` best groups can be chosen (ties: the lower index).  The `top` largest
- * allowed s are chosen; weights = s (renorm != 0: divided by the sum of the chosen + 1e-20) * scale. */
+ * allowed s are chosen; weights = s (renorm != 0: divided by the sum of the chosen + 1e-20) * scale.
+ * correction != NULL (device F32 [E]): groups and experts are chosen by s + correction (which may be negative); the weights are s without it. */
 typedef struct ntk_route_desc {
     int score;
     int groups, keep, group_top;
     int renorm;
     float scale;
+    const float* correction;
+    /* add_y != NULL: the token's row is first h[t] += add_y[t] / sqrt(mean(add_y[t]^2) + add_eps) * add_w (h is written: what the stream was still owed joins it in
+     * the router's launch, see ntk_rms_seam) */
+    const float* add_y; int ld_add; const float* add_w; float add_eps;
 } ntk_route_desc;
 int ntk_moe_route_ex(int* ids, float* wts, float* sgate, const float* h, int ldh, const float* w_router, const float* shared_gate_w, int T, int n, int E, int top,
                      const ntk_route_desc* r, void* stream);
+/* The experts of a few tokens (T <= ntk_dense_few_rows(), decoding) in two launches, without grouping: plain units U_e then D_e with the activation `act` between them,
+ *   out[t] = sum_s wts[t][s] * D_e act(U_e h[t])  (e = ids[t][s]; e >= experts: wts[t][s] * h[t])  + sgate[t] * Ds act(Us h[t])   (shared_up may be NULL; sgate NULL: 1)
+ * up [experts][ff][n], down [experts][n][ff], shared_up [shared_ff][n], shared_down [n][shared_ff], all of dtype wdtype; mid: work space F32 [T][top * ff + shared_ff].
+ * The first launch streams the chosen experts' and the shared unit's first matrices as one; the second walks a token's chosen second matrices as ONE row per output:
+ * the activations, each times its expert's weight, sit side by side in LDS (top * ff + shared_ff <= NTK_MOE_FEW_MID). */
+#define NTK_MOE_FEW_MID 36864
+typedef struct ntk_moe_few_desc {
+    float* out; int ldo;
+    const float* h; int ldh;
+    const int* ids; const float* wts; int top, experts;
+    const void* up; const void* down; int ff;
+    const void* shared_up; const void* shared_down; int shared_ff; const float* sgate;
+    int wdtype, act;
+    float* mid;
+    int T, n;
+} ntk_moe_few_desc;
+int ntk_moe_few(const ntk_moe_few_desc* d, void* stream);
 /* Stable grouping of the T*top (token, slot) pairs by expert: offsets [E+1], order [T*top] (pair index t*top+slot of every sorted row),
  * where [T*top] (sorted row of every pair). */
 int ntk_moe_group(int* offsets, int* order, int* where, const int* ids, int T, int top, int E, void* stream);
@@ -341,6 +384,10 @@ int ntk_glu_rows(float* a, int lda, const float* gu, int ldgu, int rows, int ff,
 /* out[t][:] = sum_s wts[t][s] * d[where[t*top+s]][:] + (sgate ? sgate[t] : 1) * shared[t][:] (if shared): the experts' sum on its own, for layers that norm it before
  * it joins the stream */
 int ntk_moe_sum(float* out, const float* d, const int* where, const float* wts, const float* shared, const float* sgate, int T, int top, int n, void* stream);
+/* ... with identity experts: a pair whose expert ids[t*top+s] >= n_experts adds wts[t][s] * h[t][:] (h [T] rows ldh floats apart; such a pair has no row in d).
+ * ids may be NULL (no identity experts); where == NULL: pair t*top+s is row t*top+s of d. */
+int ntk_moe_sum_ex(float* out, const float* d, const int* where, const int* ids, int n_experts, const float* h, int ldh, const float* wts, const float* shared,
+                   const float* sgate, int T, int top, int n, void* stream);
 /* x[t][:] += mix[t][:] (if mix) + sum_s wts[t][s] * d[where[t*top+s]][:] + sgate[t] * shared[t][:] (if shared) -- slots in order, one rounding sequence per token */
 int ntk_moe_combine(float* x, const float* mix, const float* d, const int* where, const float* wts, const float* shared, const float* sgate, int T, int top,
                     int n, void* stream);

@@ -34,11 +34,18 @@ struct DenseArgs {
     int T, N, K, accumulate, G, vec, xvec;   // vec: weight rows 16-byte aligned, K % 8 == 0; xvec: activation rows (and norm_w) 16-byte aligned, K % 4 == 0
     int glu_ff; float glu_limit, glu_alpha, glu_up_offset, glu_cubic;   // few-row form only: outputs f < glu_ff = gated unit of rows f (gate) and glu_ff + f (up)
     const float* norm_w; float norm_eps, norm_offset;   // few-row form only: the activation row is RMS-normed with weight (offset + norm_w) first
+    int act;                                            // NTK_ACT_*: on every output
+    const float* add_y; int ld_add; const float* add_w; float add_eps, add_mult; float* x_out; int ldxo;   // few-row form only: see ntk_dense_desc
 };
 
 __device__ __forceinline__ bool group_range(const DenseArgs& a, int g, int& r0, int& r1) {
     if (a.offsets) { r0 = a.offsets[g]; r1 = a.offsets[g + 1]; } else { r0 = 0; r1 = a.T; }
     return r1 > r0;
+}
+
+__device__ __forceinline__ float activate(float v, int act) {
+    if (act == NTK_ACT_RELU2) { const float p = fmaxf(v, 0.0f); return p * p; }
+    return v;
 }
 
 // ---------------------------------------------------------------------------------------------------------------- bf16, matrix cores
@@ -164,7 +171,7 @@ __global__ __launch_bounds__(256) void dense_mfma_kernel(const DenseArgs a) {
         for (int j = 0; j < NJ; ++j)
 #pragma unroll
             for (int r = 0; r < 4; ++r)
-                if (row + r < r1 && j * 16 < n_left) y[(long long)r * a.ldy + j * 16] = acc[i][j][r];
+                if (row + r < r1 && j * 16 < n_left) y[(long long)r * a.ldy + j * 16] = activate(acc[i][j][r], a.act);
     }
 }
 
@@ -219,7 +226,7 @@ __global__ __launch_bounds__(256) void dense_fma_kernel(const DenseArgs a) {
             const int row = row_base + ty * 4 + i, col = n_base + tx * 4 + j;
             if (row < r1 && col < a.N) {
                 float* y = a.Y + (long long)row * a.ldy + col;
-                *y = a.accumulate ? *y + acc[i][j] : acc[i][j];
+                *y = a.accumulate ? *y + acc[i][j] : activate(acc[i][j], a.act);
             }
         }
 }
@@ -230,7 +237,7 @@ __global__ __launch_bounds__(256) void dense_fma_kernel(const DenseArgs a) {
 // have arrived; one DPP reduction per row at the end.  The first weights are requested together with the activation row and the weights of its norm, so they
 // travel behind the norm's sum over the workgroup.  RW is picked so that the launch still has a few workgroups per CU.
 constexpr int kGemvRows = 8;       // up to this many rows take this form
-template <typename WT, int RW, bool GLU>
+template <typename WT, int RW, bool GLU, bool ADD>
 __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xs[];   // the activation row
     const int r = blockIdx.y;
@@ -259,23 +266,52 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
 #pragma unroll
             for (int p = 0; p < NV; ++p) u[i][p] = __builtin_nontemporal_load(reinterpret_cast<const uintx4_t*>(w[i] + k) + p);
     };
+    __shared__ float red[16];
     float ss = 0.0f;
     uintx4_t first[RW][NV];
     if (a.xvec) {
         // the row's first 4096 entries stay in registers up to the norm; they, their norm weights and the wave's first weights are requested together
         constexpr int XV = 4;
-        float4 xv[XV], nv[XV];
+        float4 xv[XV], nv[XV], yv[XV], aw[XV];
+        const float* yrow = ADD ? a.add_y + (long long)r * a.ld_add : nullptr;
 #pragma unroll
         for (int u = 0; u < XV; ++u) {
             const int k = 4 * (tid + 256 * u);
+            if constexpr (ADD) {
+                yv[u] = k < a.K ? *reinterpret_cast<const float4*>(yrow + k) : float4{0.0f, 0.0f, 0.0f, 0.0f};
+                aw[u] = k < a.K ? *reinterpret_cast<const float4*>(a.add_w + k) : float4{0.0f, 0.0f, 0.0f, 0.0f};
+            }
             xv[u] = k < a.K ? *reinterpret_cast<const float4*>(xrow + k) : float4{0.0f, 0.0f, 0.0f, 0.0f};
             nv[u] = a.norm_w && k < a.K ? *reinterpret_cast<const float4*>(a.norm_w + k) : float4{0.0f, 0.0f, 0.0f, 0.0f};
         }
         if (a.vec && lane * 8 < a.K) weights(first, lane * 8);
         for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256) *reinterpret_cast<float4*>(xs + k) = *reinterpret_cast<const float4*>(xrow + k);
         float inv = 1.0f;
+        if constexpr (ADD) {                                // what the row is still owed joins it; the first workgroup of the row leaves the sum
+            float sy = 0.0f;
+#pragma unroll
+            for (int u = 0; u < XV; ++u) { sy = fmaf(yv[u].x, yv[u].x, sy); sy = fmaf(yv[u].y, yv[u].y, sy); sy = fmaf(yv[u].z, yv[u].z, sy); sy = fmaf(yv[u].w, yv[u].w, sy); }
+            for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) sy = fmaf(yrow[k + j], yrow[k + j], sy);
+            const float iy = a.add_mult / sqrtf(block_sum(sy, red) / (float)a.K + a.add_eps);
+            float* keep = blockIdx.x == 0 ? a.x_out + (long long)r * a.ldxo : nullptr;
+#pragma unroll
+            for (int u = 0; u < XV; ++u) {
+                const int k = 4 * (tid + 256 * u);
+                if (k >= a.K) continue;
+                xv[u].x = fmaf(yv[u].x * iy, aw[u].x, xv[u].x); xv[u].y = fmaf(yv[u].y * iy, aw[u].y, xv[u].y);
+                xv[u].z = fmaf(yv[u].z * iy, aw[u].z, xv[u].z); xv[u].w = fmaf(yv[u].w * iy, aw[u].w, xv[u].w);
+                if (keep) *reinterpret_cast<float4*>(keep + k) = xv[u];
+            }
+            for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {               // (each thread rewrites what it wrote)
+                    xs[k + j] = fmaf(yrow[k + j] * iy, a.add_w[k + j], xs[k + j]);
+                    if (keep) keep[k + j] = xs[k + j];
+                }
+        }
         if (a.norm_w) {                                     // (uniform over the launch)
-            __shared__ float red[16];
 #pragma unroll
             for (int u = 0; u < XV; ++u) { ss = fmaf(xv[u].x, xv[u].x, ss); ss = fmaf(xv[u].y, xv[u].y, ss); ss = fmaf(xv[u].z, xv[u].z, ss); ss = fmaf(xv[u].w, xv[u].w, ss); }
             for (int k = 4 * (tid + 256 * XV); k < a.K; k += 4 * 256)
@@ -296,9 +332,22 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
         }
     } else {
         if (a.vec && lane * 8 < a.K) weights(first, lane * 8);
-        for (int k = tid; k < a.K; k += 256) { const float v = xrow[k]; xs[k] = v; ss = fmaf(v, v, ss); }
+        if constexpr (ADD) {
+            const float* yrow = a.add_y + (long long)r * a.ld_add;
+            float sy = 0.0f;
+            for (int k = tid; k < a.K; k += 256) { xs[k] = xrow[k]; sy = fmaf(yrow[k], yrow[k], sy); }
+            const float iy = a.add_mult / sqrtf(block_sum(sy, red) / (float)a.K + a.add_eps);
+            float* keep = blockIdx.x == 0 ? a.x_out + (long long)r * a.ldxo : nullptr;
+            for (int k = tid; k < a.K; k += 256) {
+                const float v = fmaf(yrow[k] * iy, a.add_w[k], xs[k]);
+                xs[k] = v;
+                ss = fmaf(v, v, ss);
+                if (keep) keep[k] = v;
+            }
+        } else {
+            for (int k = tid; k < a.K; k += 256) { const float v = xrow[k]; xs[k] = v; ss = fmaf(v, v, ss); }
+        }
         if (a.norm_w) {
-            __shared__ float red[16];
             ss = block_sum(ss, red);
             const float inv = 1.0f / sqrtf(ss / (float)a.K + a.norm_eps);
             for (int k = tid; k < a.K; k += 256) xs[k] = xs[k] * inv * (a.norm_offset + a.norm_w[k]);   // (each thread rewrites what it wrote)
@@ -366,12 +415,192 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(const DenseArgs a) {
                 t = gg * (1.0f / (1.0f + expf(-a.glu_alpha * zz))) * (uu + a.glu_up_offset);
             }
             float* y = a.Y + (long long)r * a.ldy + n0 + i;
-            *y = a.accumulate ? *y + t : t;
+            *y = a.accumulate ? *y + t : activate(t, a.act);
         }
     }
 }
 
+// ---------------------------------------------------------------------------------------------------------------- a few tokens' experts
+// Two launches for everything between a router and the sum of its experts (see ntk_moe_few).  Both stream weight rows like dense_gemv_kernel: a wave owns RW rows, the
+// next pass's 16 bytes per lane and row are requested before the current ones are used, the first ones ahead of the activations' way into LDS.
+struct MoeFewArgs {
+    float* out; int ldo;
+    const float* h; int ldh;
+    const int* ids; const float* wts; int top, experts;
+    const void *up, *down, *shared_up, *shared_down; int ff, shared_ff;
+    const float* sgate;
+    int act; float* mid; int n, vec;
+};
+
+template <typename WT> struct WeightPiece {                  // eight weights of a row
+    static constexpr int NV = sizeof(WT) == 2 ? 1 : 2;
+    uintx4_t u[NV];
+    __device__ __forceinline__ void load(const WT* p) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) u[i] = __builtin_nontemporal_load(reinterpret_cast<const uintx4_t*>(p) + i);
+    }
+    __device__ __forceinline__ void clear() {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) u[i] = uintx4_t{0u, 0u, 0u, 0u};
+    }
+    __device__ __forceinline__ float dot(const float* x, float s) const {      // s + the eight products, k ascending; x 16-byte aligned
+        const float4 x0 = *reinterpret_cast<const float4*>(x), x1 = *reinterpret_cast<const float4*>(x + 4);
+        const float xv[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+        if constexpr (sizeof(WT) == 2) {
+            const uint32_t w[4] = {u[0].x, u[0].y, u[0].z, u[0].w};
+#pragma unroll
+            for (int j = 0; j < 4; ++j) { s = fmaf(__uint_as_float(w[j] << 16), xv[2 * j], s); s = fmaf(__uint_as_float(w[j] & 0xffff0000u), xv[2 * j + 1], s); }
+        } else {
+#pragma unroll
+            for (int p = 0; p < 2; ++p) {
+                s = fmaf(__uint_as_float(u[p].x), xv[4 * p], s); s = fmaf(__uint_as_float(u[p].y), xv[4 * p + 1], s);
+                s = fmaf(__uint_as_float(u[p].z), xv[4 * p + 2], s); s = fmaf(__uint_as_float(u[p].w), xv[4 * p + 3], s);
+            }
+        }
+        return s;
+    }
+};
+template <typename WT> __device__ __forceinline__ float weight_value(const WT* p) {
+    if constexpr (sizeof(WT) == 2) return bf2f(*p); else return *p;
+}
+
+// mid[t][slot * ff + f] = act(U_e h)[f] for the token's chosen experts, then the shared unit's; grid (rows / (4 RW), T)
+template <typename WT, int RW>
+__global__ __launch_bounds__(256) void moe_few_up_kernel(const MoeFewArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];   // the token's row
+    const int t = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int routed = a.top * a.ff, rows = routed + a.shared_ff, m0 = (blockIdx.x * 4 + wave) * RW;
+    const int* ids = a.ids + (long long)t * a.top;
+    const WT* w[RW];
+    bool any = false;
+#pragma unroll
+    for (int i = 0; i < RW; ++i) {                            // rows of identity experts and rows past the end: nothing to read
+        const int m = m0 + i;
+        w[i] = nullptr;
+        if (m < routed) {
+            const int e = ids[m / a.ff];
+            if (e >= 0 && e < a.experts) w[i] = (const WT*)a.up + ((long long)e * a.ff + m % a.ff) * a.n;
+        } else if (m < rows) {
+            w[i] = (const WT*)a.shared_up + (long long)(m - routed) * a.n;
+        }
+        any = any || w[i];
+    }
+    WeightPiece<WT> cur[RW], next[RW];
+    auto request = [&](WeightPiece<WT>(&p)[RW], int k) {
+#pragma unroll
+        for (int i = 0; i < RW; ++i) { if (w[i]) p[i].load(w[i] + k); else p[i].clear(); }
+    };
+    if (a.vec && lane * 8 < a.n) request(cur, lane * 8);
+    const float* x = a.h + (long long)t * a.ldh;
+    if (a.vec)
+        for (int k = 4 * tid; k < a.n; k += 4 * 256) *reinterpret_cast<float4*>(xs + k) = *reinterpret_cast<const float4*>(x + k);
+    else
+        for (int k = tid; k < a.n; k += 256) xs[k] = x[k];
+    __syncthreads();
+    if (!any) return;                                         // (uniform over the wave)
+    float s[RW];
+#pragma unroll
+    for (int i = 0; i < RW; ++i) s[i] = 0.0f;
+    if (a.vec) {
+        for (int k = lane * 8; k < a.n; k += 512) {
+            if (k + 512 < a.n) request(next, k + 512);
+#pragma unroll
+            for (int i = 0; i < RW; ++i) { s[i] = cur[i].dot(xs + k, s[i]); cur[i] = next[i]; }
+        }
+    } else {
+        for (int k = lane; k < a.n; k += 64)
+#pragma unroll
+            for (int i = 0; i < RW; ++i)
+                if (w[i]) s[i] = fmaf(weight_value(w[i] + k), xs[k], s[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < RW; ++i) {
+        s[i] = wave_sum_lane63(s[i]);
+        if (lane == 63 && w[i]) a.mid[(long long)t * rows + m0 + i] = activate(s[i], a.act);
+    }
+}
+
+// out[t][i] = one row of weights [D_e0[i] | D_e1[i] | ... | Ds[i]] against the activations side by side, each times its expert's weight; grid (n / (4 RW), T)
+template <typename WT, int RW>
+__global__ __launch_bounds__(256) void moe_few_down_kernel(const MoeFewArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];   // [top * ff + shared_ff] weighted activations
+    const int t = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int routed = a.top * a.ff, K = routed + a.shared_ff, i0 = (blockIdx.x * 4 + wave) * RW;
+    const int* ids = a.ids + (long long)t * a.top;
+    const float* wts = a.wts + (long long)t * a.top;
+    int row[RW];
+#pragma unroll
+    for (int i = 0; i < RW; ++i) row[i] = min(i0 + i, a.n - 1);     // (rows past the end re-read the last one and are not stored)
+    // where a lane stands in the concatenated row: segment (slot; `top` = the shared unit) and place in it
+    int slot = 0, off = 0;
+    auto settle = [&]() { while (slot < a.top && off >= a.ff) { off -= a.ff; ++slot; } };
+    WeightPiece<WT> cur[RW], next[RW];
+    auto request = [&](WeightPiece<WT>(&p)[RW]) {
+        const WT* base = nullptr;
+        long long step = 0;
+        if (slot < a.top) {
+            const int e = ids[slot];
+            if (e >= 0 && e < a.experts) { base = (const WT*)a.down + (long long)e * a.n * a.ff + off; step = a.ff; }
+        } else if (off < a.shared_ff) {
+            base = (const WT*)a.shared_down + off; step = a.shared_ff;
+        }
+#pragma unroll
+        for (int i = 0; i < RW; ++i) { if (base) p[i].load(base + row[i] * step); else p[i].clear(); }
+    };
+    if (a.vec) { off = lane * 8; settle(); request(cur); }
+    for (int m = tid; m < K; m += 256) {
+        const int sl = m / a.ff;                              // (beyond the routed part: >= top)
+        float wt = a.sgate ? a.sgate[t] : 1.0f;
+        bool live = true;
+        if (m < routed) { const int e = ids[sl]; wt = wts[sl]; live = e >= 0 && e < a.experts; }
+        xs[m] = live ? a.mid[(long long)t * K + m] * wt : 0.0f;     // (an identity expert's part of the work space is not written)
+    }
+    __syncthreads();
+    if (i0 >= a.n) return;                                    // (uniform over the wave)
+    float s[RW];
+#pragma unroll
+    for (int i = 0; i < RW; ++i) s[i] = 0.0f;
+    if (a.vec) {
+        for (int k = lane * 8; k < K; k += 512) {
+            if (k + 512 < K) { off += 512; settle(); request(next); }
+#pragma unroll
+            for (int i = 0; i < RW; ++i) { s[i] = cur[i].dot(xs + k, s[i]); cur[i] = next[i]; }
+        }
+    } else {
+        for (int k = lane; k < K; k += 64) {
+            const WT* base;
+            long long step;
+            if (k < routed) {
+                const int e = ids[k / a.ff];
+                if (e < 0 || e >= a.experts) continue;
+                base = (const WT*)a.down + (long long)e * a.n * a.ff + k % a.ff; step = a.ff;
+            } else {
+                base = (const WT*)a.shared_down + (k - routed); step = a.shared_ff;
+            }
+#pragma unroll
+            for (int i = 0; i < RW; ++i) s[i] = fmaf(weight_value(base + row[i] * step), xs[k], s[i]);
+        }
+    }
+    float ident = 0.0f;                                       // the weights of the token's identity experts
+    for (int sl = 0; sl < a.top; ++sl)
+        if (ids[sl] >= a.experts) ident += wts[sl];
+#pragma unroll
+    for (int i = 0; i < RW; ++i) {
+        s[i] = wave_sum_lane63(s[i]);
+        if (lane == 63 && i0 + i < a.n) a.out[(long long)t * a.ldo + i0 + i] = ident != 0.0f ? fmaf(ident, a.h[(long long)t * a.ldh + i0 + i], s[i]) : s[i];
+    }
+}
+
 template <typename WT>
+static void launch_moe_few(const MoeFewArgs& a, int T, hipStream_t s) {
+    const int rows = a.top * a.ff + a.shared_ff;
+    constexpr int RW = 2;
+    const dim3 gu((rows + 4 * RW - 1) / (4 * RW), T), gd((a.n + 4 * RW - 1) / (4 * RW), T);
+    hipLaunchKernelGGL((moe_few_up_kernel<WT, RW>), gu, dim3(256), ((size_t)a.n * 4 + 15) & ~(size_t)15, s, a);
+    hipLaunchKernelGGL((moe_few_down_kernel<WT, RW>), gd, dim3(256), ((size_t)rows * 4 + 15) & ~(size_t)15, s, a);
+}
+
+template <typename WT, bool ADD>
 static void launch_gemv(const DenseArgs& a, int rows, hipStream_t s) {
     const size_t lds = ((size_t)a.K * 4 + 15) & ~(size_t)15;
     // Rows per wave, measured over layer-like shapes (2048 .. 64000 outputs of 768 .. 4096 inputs, 1 .. 6 activation rows): two rows per wave are
@@ -383,16 +612,16 @@ static void launch_gemv(const DenseArgs& a, int rows, hipStream_t s) {
     if (a.glu_ff > 0) {
         const int out = work >= 4 * 8 * 512 ? 4 : work >= 4 * 4 * 512 ? 2 : 1;   // (gate, up) pairs per wave
         const dim3 grid((a.glu_ff + 4 * out - 1) / (4 * out), rows, 1);
-        if (out == 4) hipLaunchKernelGGL((dense_gemv_kernel<WT, 8, true>), grid, dim3(256), lds, s, a);
-        else if (out == 2) hipLaunchKernelGGL((dense_gemv_kernel<WT, 4, true>), grid, dim3(256), lds, s, a);
-        else hipLaunchKernelGGL((dense_gemv_kernel<WT, 2, true>), grid, dim3(256), lds, s, a);
+        if (out == 4) hipLaunchKernelGGL((dense_gemv_kernel<WT, 8, true, ADD>), grid, dim3(256), lds, s, a);
+        else if (out == 2) hipLaunchKernelGGL((dense_gemv_kernel<WT, 4, true, ADD>), grid, dim3(256), lds, s, a);
+        else hipLaunchKernelGGL((dense_gemv_kernel<WT, 2, true, ADD>), grid, dim3(256), lds, s, a);
         return;
     }
     const dim3 grid((a.N + 4 * rw - 1) / (4 * rw), rows, 1);
-    if (rw == 8) hipLaunchKernelGGL((dense_gemv_kernel<WT, 8, false>), grid, dim3(256), lds, s, a);
-    else if (rw == 4) hipLaunchKernelGGL((dense_gemv_kernel<WT, 4, false>), grid, dim3(256), lds, s, a);
-    else if (rw == 2) hipLaunchKernelGGL((dense_gemv_kernel<WT, 2, false>), grid, dim3(256), lds, s, a);
-    else hipLaunchKernelGGL((dense_gemv_kernel<WT, 1, false>), grid, dim3(256), lds, s, a);
+    if (rw == 8) hipLaunchKernelGGL((dense_gemv_kernel<WT, 8, false, ADD>), grid, dim3(256), lds, s, a);
+    else if (rw == 4) hipLaunchKernelGGL((dense_gemv_kernel<WT, 4, false, ADD>), grid, dim3(256), lds, s, a);
+    else if (rw == 2) hipLaunchKernelGGL((dense_gemv_kernel<WT, 2, false, ADD>), grid, dim3(256), lds, s, a);
+    else hipLaunchKernelGGL((dense_gemv_kernel<WT, 1, false, ADD>), grid, dim3(256), lds, s, a);
 }
 
 }  // namespace ntk
@@ -407,9 +636,12 @@ int ntk_dense(const ntk_dense_desc* d, void* stream) {
     if (d->rows && d->row_div <= 0) return NTK_E_SHAPE;
     if (d->glu_ff > 0 && (d->T > kGemvRows || d->N != 2 * d->glu_ff || d->accumulate)) return NTK_E_SHAPE;
     if (d->norm_w && d->T > kGemvRows) return NTK_E_SHAPE;
+    if ((d->act != NTK_ACT_NONE && d->act != NTK_ACT_RELU2) || (d->act && (d->accumulate || d->glu_ff > 0))) return NTK_E_SHAPE;
+    if (d->add_y && (!d->add_w || !d->x_out)) return NTK_E_NULL;
+    if (d->add_y && (d->T > kGemvRows || d->rows || d->offsets || d->ld_add < d->K || d->ldxo < d->K || d->x_out == d->X || d->x_out == d->add_y)) return NTK_E_SHAPE;
     if (d->T == 0) return NTK_OK;
     const int G = d->offsets ? d->G : 1;
-    DenseArgs a{d->Y, d->ldy, d->X, d->ldx, d->W, d->wstride, d->offsets, d->rows, d->rows ? d->row_div : 1, d->T, d->N, d->K, d->accumulate, G, 0, 0, 0, 0.0f, 0.0f, 0.0f, 0.0f, nullptr, 0.0f, 0.0f};
+    DenseArgs a{d->Y, d->ldy, d->X, d->ldx, d->W, d->wstride, d->offsets, d->rows, d->rows ? d->row_div : 1, d->T, d->N, d->K, d->accumulate, G, 0, 0, 0, 0.0f, 0.0f, 0.0f, 0.0f, nullptr, 0.0f, 0.0f, d->act, nullptr, 0, nullptr, 0.0f, 0.0f, nullptr, 0};
     hipStream_t s = resolve_stream(stream);
     if (d->T <= kGemvRows) {
         if ((size_t)d->K * 4 > 160 * 1024 - 1024) return NTK_E_SHAPE;
@@ -417,8 +649,15 @@ int ntk_dense(const ntk_dense_desc* d, void* stream) {
         a.norm_w = d->norm_w; a.norm_eps = d->norm_eps; a.norm_offset = d->norm_offset;
         a.vec = (d->K % 8 == 0) && !((uintptr_t)d->W & 15) && !((d->wstride * (d->wdtype == NTK_DT_BF16 ? 2 : 4)) & 15);
         a.xvec = (d->K % 4 == 0) && (d->ldx % 4 == 0) && !((uintptr_t)d->X & 15) && !((uintptr_t)d->norm_w & 15);
-        if (d->wdtype == NTK_DT_BF16) launch_gemv<uint16_t>(a, d->T, s);
-        else launch_gemv<float>(a, d->T, s);
+        if (d->add_y) {
+            a.add_y = d->add_y; a.ld_add = d->ld_add; a.add_w = d->add_w; a.add_eps = d->add_eps; a.add_mult = d->add_mult; a.x_out = d->x_out; a.ldxo = d->ldxo;
+            a.xvec = a.xvec && (d->ld_add % 4 == 0) && (d->ldxo % 4 == 0) && !(((uintptr_t)d->add_y | (uintptr_t)d->add_w | (uintptr_t)d->x_out) & 15);
+            if (d->wdtype == NTK_DT_BF16) launch_gemv<uint16_t, true>(a, d->T, s);
+            else launch_gemv<float, true>(a, d->T, s);
+            return last_launch_status();
+        }
+        if (d->wdtype == NTK_DT_BF16) launch_gemv<uint16_t, false>(a, d->T, s);
+        else launch_gemv<float, false>(a, d->T, s);
         return last_launch_status();
     }
     if (d->wdtype == NTK_DT_BF16) {
@@ -443,6 +682,27 @@ int ntk_dense(const ntk_dense_desc* d, void* stream) {
         const dim3 grid((d->N + TN - 1) / TN, (d->T + TM - 1) / TM, G);
         hipLaunchKernelGGL(dense_fma_kernel, grid, dim3(256), 0, s, a);
     }
+    return last_launch_status();
+}
+
+int ntk_moe_few(const ntk_moe_few_desc* d, void* stream) {
+    if (!d || !d->out || !d->h || !d->ids || !d->wts || !d->up || !d->down || !d->mid || (d->shared_ff > 0 && (!d->shared_up || !d->shared_down))) return NTK_E_NULL;
+    if (d->wdtype != NTK_DT_BF16 && d->wdtype != NTK_DT_F32) return NTK_E_DTYPE;
+    if (d->act != NTK_ACT_NONE && d->act != NTK_ACT_RELU2) return NTK_E_SHAPE;
+    if (d->T < 0 || d->T > kGemvRows || d->n <= 0 || d->top <= 0 || d->experts <= 0 || d->ff <= 0 || d->shared_ff < 0 || d->ldo < d->n || d->ldh < d->n) return NTK_E_SHAPE;
+    if ((long long)d->top * d->ff + d->shared_ff > NTK_MOE_FEW_MID || d->n > NTK_MOE_FEW_MID) return NTK_E_SHAPE;
+    if (d->T == 0) return NTK_OK;
+    MoeFewArgs a{d->out, d->ldo, d->h, d->ldh, d->ids, d->wts, d->top, d->experts, d->up, d->down, d->shared_up, d->shared_down, d->ff, d->shared_ff, d->sgate, d->act, d->mid, d->n, 0};
+    a.vec = d->n % 8 == 0 && d->ff % 8 == 0 && d->shared_ff % 8 == 0 && d->ldh % 4 == 0 &&
+            !(((uintptr_t)d->h | (uintptr_t)d->up | (uintptr_t)d->down | (uintptr_t)d->shared_up | (uintptr_t)d->shared_down) & 15);
+    static bool raised = false;     // (idempotent: a race sets the same attributes twice)
+    if (!raised) {
+        const void* fn[] = {(const void*)moe_few_up_kernel<uint16_t, 2>, (const void*)moe_few_up_kernel<float, 2>, (const void*)moe_few_down_kernel<uint16_t, 2>, (const void*)moe_few_down_kernel<float, 2>};
+        for (const void* f : fn) NTK_HIP_TRY(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, NTK_MOE_FEW_MID * 4));
+        raised = true;
+    }
+    if (d->wdtype == NTK_DT_BF16) launch_moe_few<uint16_t>(a, d->T, resolve_stream(stream));
+    else launch_moe_few<float>(a, d->T, resolve_stream(stream));
     return last_launch_status();
 }
 

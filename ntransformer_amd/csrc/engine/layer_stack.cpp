@@ -39,11 +39,19 @@ static StackForm dense_parallel_form() {
     f.rot_halves = true; f.blended_rotation = true; f.learned_sinks = true; f.attention_gate = true; f.attention_head_gate = true; f.whole_qk_norm = true;
     return f;
 }
+static StackForm post_norm_form() {
+    StackForm f;
+    f.post_norm = true; f.loop_projection = false; f.clipped_glu = false; f.plain_experts = true; f.router_correction = true; f.router_renorm = false; f.group_top = 1;
+    f.attention_gate = true; f.head_qk_norm = true; f.raw_key_values = true; f.distance_slopes = true; f.latent_plain = true; f.latent_head_gate = true;
+    return f;
+}
+static constexpr double kPositionBase = 10000.0;   // of the sinusoidal position vector
 // what the gated form's mechanisms fix
 static constexpr float kGeluAlpha = 1.5957691216057308f;   // 2 sqrt(2 / pi): 0.5 (1 + tanh y) = sigmoid(2 y)
 static constexpr float kGeluCubic = 0.044715f;
 static constexpr float kDeltaDecayRate = 0.6065306597126334f;   // exp(-1/2): w = exp(-rate * sigmoid(.))
 static constexpr float kUnitKeyEps = 1e-6f;
+static FamilyRegistrar reg_gibevik("Gibevik", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(post_norm_form())); });
 static FamilyRegistrar reg_zalazen("Zalazen", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(dense_parallel_form())); });
 static FamilyRegistrar reg_fifotar("Fifotar", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(scaled_form())); });
 static FamilyRegistrar reg_tubazen("Tubazen", [] { return std::unique_ptr<SequenceModel>(new LayerStackModel(gated_form())); });
@@ -97,9 +105,20 @@ int LayerStackModel::parse_mixer(const Json& L, const std::string& type, LatentM
     const Json& mx = L.at("mixer");
     const std::string where = "mixer '" + type + "'";
     if (!mx.is_object()) return fail(NTK_E_FORMAT, where + ": no 'mixer' object");
-    if (!need_int(mx, "heads", m.heads, err_, where) || !need_int(mx, "dim", m.dim, err_, where) || !need_int(mx, "rot_dim", m.rot_dim, err_, where) ||
-        !need_int(mx, "vdim", m.vdim, err_, where) || !need_int(mx, "kv_rank", m.kv_rank, err_, where))
+    if (!need_int(mx, "heads", m.heads, err_, where) || !need_int(mx, "dim", m.dim, err_, where) || !need_int(mx, "vdim", m.vdim, err_, where) ||
+        !need_int(mx, "kv_rank", m.kv_rank, err_, where))
         return NTK_E_FORMAT;
+    if (form_.latent_plain) {
+        m.head_gate = form_.latent_head_gate;
+        if (!mx.at("scale").is_number()) return fail(NTK_E_FORMAT, where + ": 'scale' is missing");
+        m.scale = (float)mx.at("scale").number();
+        if (mx.at("kv_from").is_number()) {
+            m.kv_from = (int)mx.at("kv_from").integer();
+            if (m.kv_from < 0) return fail(NTK_E_FORMAT, where + ": kv_from must name a layer");
+        }
+        return NTK_OK;
+    }
+    if (!need_int(mx, "rot_dim", m.rot_dim, err_, where)) return NTK_E_FORMAT;
     if (type == "latent_attention") {
         if (!need_int(mx, "q_rank", m.q_rank, err_, where)) return NTK_E_FORMAT;
     } else {
@@ -172,6 +191,25 @@ int LayerStackModel::parse_window(const Json& L, WindowMixer& m) {
     if (form_.dense_parallel && mx.at("kv_from").is_number()) {
         m.kv_from = (int)mx.at("kv_from").integer();
         if (m.kv_from < 0) return fail(NTK_E_FORMAT, where + ": kv_from must name a layer");
+    }
+    if (form_.head_qk_norm) {
+        m.head_norm = true;
+        if (mx.at("q_temp").is_object()) {
+            m.temp_coef = (float)mx.at("q_temp").at("coef").number(0.0);
+            m.temp_every = mx.at("q_temp").at("every").number(1.0);
+            if (!(m.temp_every > 0.0)) return fail(NTK_E_FORMAT, where + ": q_temp.every must be positive");
+        }
+    }
+    if (form_.raw_key_values) {
+        m.raw_key_values = true;
+        if (m.vdim != m.dim) return fail(NTK_E_FORMAT, where + ": values that are keys have the keys' size: vdim must equal dim");
+    }
+    if (form_.distance_slopes) {
+        std::vector<float> sl((size_t)m.heads);
+        for (int h = 0; h < m.heads; ++h) sl[(size_t)h] = (float)std::exp2(-8.0 * (h + 1) / m.heads);
+        m.slopes = (float*)dev_alloc(sl.size() * sizeof(float));
+        if (!m.slopes) return fail(NTK_E_NOMEM, "out of device memory");
+        nt_hip_memcpy_h2d(m.slopes, sl.data(), sl.size() * sizeof(float));
     }
     m.softcap = (float)mx.at("softcap").number(0.0);
     if (m.softcap < 0.0f) return fail(NTK_E_FORMAT, where + ": 'softcap' must be positive");
@@ -269,11 +307,11 @@ int LayerStackModel::parse_parallel(const Json& L, ParallelMixer& m) {
 
 int LayerStackModel::parse_mlp(const Json& ml, const std::string& where, StackLayer& S) {
     const std::string kind = ml.at("kind").is_string() ? ml.at("kind").str : "moe";
-    if (kind == "dense" && (form_.scaled || form_.dense_parallel)) {
+    if (kind == "dense" && (form_.scaled || form_.dense_parallel || form_.post_norm)) {
         S.mlp_kind = kMlpUnit;
         if (!need_int(ml, "ff", S.cff.ff, err_, where)) return NTK_E_FORMAT;
         S.cff.limit = INFINITY;
-        if (form_.dense_parallel) return NTK_OK;
+        if (!form_.clipped_glu) return NTK_OK;
         S.cff.limit = ml.at("limit").is_number() ? (float)ml.at("limit").number() : INFINITY;
         if (!(S.cff.limit > 0.0f)) return fail(NTK_E_FORMAT, where + ": 'limit' must be positive");
         return NTK_OK;
@@ -290,19 +328,25 @@ int LayerStackModel::parse_mlp(const Json& ml, const std::string& where, StackLa
     const Json& rt = ml.at("router");
     if (!need_int(rt, "experts", M.experts, err_, where) || !need_int(rt, "top", M.top, err_, where) || !need_int(ml.at("expert"), "ff", M.routed.ff, err_, where))
         return NTK_E_FORMAT;
-    if (M.top > M.experts || M.experts > 255) return fail(NTK_E_FORMAT, where + ": top <= experts <= 255 is required");
+    if (form_.router_correction && rt.at("identity").is_number()) {
+        M.identity = (int)rt.at("identity").integer();
+        if (M.identity < 0) return fail(NTK_E_FORMAT, where + ": router.identity must not be negative");
+    }
+    const int choices = M.experts + M.identity;
+    if (M.top > choices || choices > 255) return fail(NTK_E_FORMAT, where + ": top <= experts (with identity experts) <= 255 is required");
     M.route.score = form_.router_score;
     M.route.renorm = form_.router_renorm ? 1 : 0;
     M.route.scale = (float)rt.at("scale").number(1.0);
     M.route.groups = 1; M.route.keep = 1; M.route.group_top = form_.group_top;
-    if (rt.has("groups")) {
+    if (rt.at("groups").is_object()) {
         if (!need_int(rt.at("groups"), "count", M.route.groups, err_, where + " groups") || !need_int(rt.at("groups"), "keep", M.route.keep, err_, where + " groups")) return NTK_E_FORMAT;
-        if (M.experts % M.route.groups || M.route.keep > M.route.groups || (long long)M.route.keep * (M.experts / M.route.groups) < M.top)
+        if (choices % M.route.groups || M.route.keep > M.route.groups || (long long)M.route.keep * (choices / M.route.groups) < M.top)
             return fail(NTK_E_FORMAT, where + ": groups must divide the experts and the kept groups must hold 'top' experts");
     }
     if (form_.clipped_glu) { M.glu_alpha = kGluAlpha; M.glu_up_offset = 1.0f; M.routed.limit = (float)ml.at("expert").at("limit").number(); }
     else { M.glu_alpha = 1.0f; M.glu_up_offset = 0.0f; M.routed.limit = INFINITY; }
-    M.has_shared = ml.has("shared");
+    M.routed.plain = M.shared.plain = form_.plain_experts;
+    M.has_shared = ml.at("shared").is_object();
     if (M.has_shared) {
         if (!need_int(ml.at("shared"), "ff", M.shared.ff, err_, where + " shared")) return NTK_E_FORMAT;
         M.shared.limit = form_.clipped_glu ? (float)ml.at("shared").at("limit").number() : INFINITY;
@@ -333,6 +377,7 @@ int LayerStackModel::parse(const ModelFolder& f) {
         if (logit_softcap_ < 0.0f) return fail(NTK_E_FORMAT, "config: logit_softcap must be positive");
         norm_offset_ = 0.0f;
     }
+    if (form_.post_norm) norm_offset_ = 0.0f;
     if (form_.dense_parallel) {
         const Json& e = c.at("embedding");
         embed_scale_ = (float)e.at("scale").number(1.0);
@@ -355,7 +400,10 @@ int LayerStackModel::parse(const ModelFolder& f) {
         StackLayer& S = layers_[i];
         S.type = L.at("type").str;
         // which mixers a form lists: the parallel form's layers read two norms of one input, so its mixers are the latent kinds it was built around
-        if (form_.dense_parallel && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
+        if (form_.post_norm && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
+        else if (form_.post_norm && S.type == "latent_attention") { S.mixer = kMixLatent; LS_TRY(parse_mixer(L, S.type, S.mix)); }
+        else if (form_.post_norm) return fail(NTK_E_FORMAT, "layer " + std::to_string(i) + ": unknown mixer type '" + S.type + "'");
+        else if (form_.dense_parallel && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
         else if (form_.dense_parallel) return fail(NTK_E_FORMAT, "layer " + std::to_string(i) + ": unknown mixer type '" + S.type + "'");
         else if (form_.scaled && S.type == "attention") { S.mixer = kMixWindow; LS_TRY(parse_window(L, S.att)); }
         else if (form_.scaled && S.type == "latent_attention") { S.mixer = kMixLatent; LS_TRY(parse_mixer(L, S.type, S.mix)); }
@@ -375,13 +423,20 @@ int LayerStackModel::parse(const ModelFolder& f) {
     // the order of layer runs
     const int n = (int)layers_.size();
     runs_.clear();
-    has_loop_ = c.has("loop") && !form_.gated && !form_.scaled && !form_.dense_parallel;   // (the gated form's depth weights are per layer: it has no repeated span; the other two list none)
+    has_loop_ = c.has("loop") && !form_.gated && !form_.scaled && !form_.dense_parallel && !form_.post_norm;   // (the gated form's depth weights are per layer: it has no repeated span; the others list none)
     for (size_t i = 0; i < layers_.size(); ++i) {   // a layer that reads another one's cache rows: an earlier layer with rows of its own, laid out alike
-        const int j = layers_[i].att.kv_from;
+        const int j = layers_[i].kv_from();
         if (j < 0) continue;
         const std::string li = "layer " + std::to_string(i);
         if (j >= (int)i) return fail(NTK_E_FORMAT, li + ": kv_from must name an earlier layer");
-        const WindowMixer &a = layers_[i].att, &b = layers_[(size_t)j].att;
+        const StackLayer& src = layers_[(size_t)j];
+        if (src.mixer != layers_[i].mixer) return fail(NTK_E_FORMAT, li + ": kv_from names a layer with another kind of mixer");
+        if (layers_[i].mixer == kMixLatent) {
+            if (src.mix.kv_from >= 0) return fail(NTK_E_FORMAT, li + ": kv_from names a layer without latents of its own");
+            if (src.mix.row() != layers_[i].mix.row() || src.mix.kv_rank != layers_[i].mix.kv_rank) return fail(NTK_E_FORMAT, li + ": kv_rank must equal that of the layer whose latents it reads");
+            continue;
+        }
+        const WindowMixer &a = layers_[i].att, &b = src.att;
         if (b.kv_from >= 0) return fail(NTK_E_FORMAT, li + ": kv_from names a layer without keys and values of its own");
         if (a.kv_heads != b.kv_heads || a.dim != b.dim || a.vdim != b.vdim) return fail(NTK_E_FORMAT, li + ": kv_heads, dim and vdim must equal those of the layer whose keys and values it reads");
     }
@@ -606,16 +661,21 @@ int LayerStackModel::upload_mixer(const ModelFolder& f, const std::string& p, in
         WindowMixer& m = L.att;
         const bool own = m.kv_from < 0;
         std::vector<std::string> names = {p + "mix.q"};
-        if (own) { names.push_back(p + "mix.k"); names.push_back(p + "mix.v"); }
+        if (own) names.push_back(p + "mix.k");
+        if (own && !m.raw_key_values) names.push_back(p + "mix.v");
         if (m.gated) names.push_back(p + "mix.g");
         LS_TRY(upload_matrix(f, names, W, m.in));
         m.k_off = m.heads * m.maps * m.dim;
         m.v_off = m.k_off + (own ? m.kv_heads * m.maps * m.dim : 0);
-        m.g_off = m.v_off + (own ? m.kv_heads * m.vdim : 0);
+        m.g_off = m.v_off + (own && !m.raw_key_values ? m.kv_heads * m.vdim : 0);
         if (own && f.tensor(p + "mix.k")->shape[0] != m.v_off - m.k_off) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.k' does not have kv_heads * maps * dim rows");
         if (form_.whole_qk_norm) {
             LS_TRY(upload_vector(f, p + "mix.q.norm", m.k_off, &m.q_norm));
             if (own) LS_TRY(upload_vector(f, p + "mix.k.norm", m.v_off - m.k_off, &m.k_norm));
+        }
+        if (m.head_norm) {
+            LS_TRY(upload_vector(f, p + "mix.q.norm", m.dim, &m.q_norm));
+            if (own) LS_TRY(upload_vector(f, p + "mix.k.norm", m.dim, &m.k_norm));
         }
         if (form_.learned_sinks) LS_TRY(upload_vector(f, p + "mix.sink", m.heads, &m.sinks));
         if (m.v_mix && !m.v_source) LS_TRY(read_scalar(f, p + "mix.vmix", &m.v_blend));
@@ -706,17 +766,19 @@ int LayerStackModel::upload_mixer(const ModelFolder& f, const std::string& p, in
     LatentMixer& m = L.mix;
     const int hq = m.heads * m.qd(), hv = m.heads * m.vdim;
     const std::string first = m.q_rank ? p + "mix.dq" : p + "mix.q";
-    LS_TRY(upload_matrix(f, {first, p + "mix.dkv", p + "mix.g"}, W, m.in));
+    const bool own = m.kv_from < 0;
+    LS_TRY(upload_matrix(f, own ? std::vector<std::string>{first, p + "mix.dkv", p + "mix.g"} : std::vector<std::string>{first, p + "mix.g"}, W, m.in));
     m.q_off = 0;
     m.kv_off = m.q_rank ? m.q_rank : hq;
-    m.g_off = m.kv_off + m.row();
+    m.g_off = m.kv_off + (own ? m.row() : 0);
+    if (f.tensor(first)->shape[0] != m.kv_off) return fail(NTK_E_SHAPE, li + ": the mixer's query projection does not have the configured size");
     if (m.in.out_f != m.g_off + (m.head_gate ? m.heads : hv)) return fail(NTK_E_SHAPE, li + ": the mixer's input projections do not have the configured sizes");
     if (m.q_rank) {
         LS_TRY(upload_vector(f, p + "mix.dq.norm", m.q_rank, &m.q_norm));
         LS_TRY(upload_matrix(f, {p + "mix.uq"}, m.q_rank, m.uq));
         if (m.uq.out_f != hq) return fail(NTK_E_SHAPE, "tensor '" + p + "mix.uq' does not have heads * (dim + rot_dim) rows");
     }
-    LS_TRY(upload_vector(f, p + "mix.dkv.norm", m.kv_rank, &m.kv_norm));
+    if (own) LS_TRY(upload_vector(f, p + "mix.dkv.norm", m.kv_rank, &m.kv_norm));
     LS_TRY(upload_matrix(f, {p + "mix.uk"}, m.kv_rank, m.uk));
     LS_TRY(upload_matrix(f, {p + "mix.uv"}, m.kv_rank, m.uv));
     LS_TRY(upload_matrix(f, {p + "mix.o"}, hv, m.o));
@@ -743,19 +805,24 @@ int LayerStackModel::upload_mlp(const ModelFolder& f, const std::string& p, int 
         return upload_vector(f, p + "mlp.act", 4, &D.act);
     }
     MoeFeedForward& M = L.mlp;
-    LS_TRY(upload_vector(f, p + "mlp.router", (int64_t)M.experts * W, &M.router));
+    LS_TRY(upload_vector(f, p + "mlp.router", (int64_t)(M.experts + M.identity) * W, &M.router));
+    if (form_.router_correction) {
+        LS_TRY(upload_vector(f, p + "mlp.correction", M.experts + M.identity, &M.correction));
+        M.route.correction = M.correction;
+    }
     std::vector<std::string> gu, dn;
     for (int e = 0; e < M.experts; ++e) {
         const std::string q = p + "mlp.e" + std::to_string(e) + ".";
-        gu.push_back(q + "gate"); gu.push_back(q + "up"); dn.push_back(q + "down");
+        if (!M.routed.plain) gu.push_back(q + "gate");
+        gu.push_back(q + "up"); dn.push_back(q + "down");
     }
     LS_TRY(upload_matrix(f, gu, W, M.routed.gate_up, M.experts));
     LS_TRY(upload_matrix(f, dn, M.routed.ff, M.routed.down, M.experts));
-    if (M.routed.gate_up.out_f != 2 * M.routed.ff || M.routed.down.out_f != W) return fail(NTK_E_SHAPE, li + ": expert matrices do not have the configured sizes");
+    if (M.routed.gate_up.out_f != M.routed.in_rows() || M.routed.down.out_f != W) return fail(NTK_E_SHAPE, li + ": expert matrices do not have the configured sizes");
     if (M.has_shared) {
-        LS_TRY(upload_matrix(f, {p + "mlp.shared.gate", p + "mlp.shared.up"}, W, M.shared.gate_up));
+        LS_TRY(upload_matrix(f, M.shared.plain ? std::vector<std::string>{p + "mlp.shared.up"} : std::vector<std::string>{p + "mlp.shared.gate", p + "mlp.shared.up"}, W, M.shared.gate_up));
         LS_TRY(upload_matrix(f, {p + "mlp.shared.down"}, M.shared.ff, M.shared.down));
-        if (M.shared.gate_up.out_f != 2 * M.shared.ff || M.shared.down.out_f != W) return fail(NTK_E_SHAPE, li + ": shared expert matrices do not have the configured sizes");
+        if (M.shared.gate_up.out_f != M.shared.in_rows() || M.shared.down.out_f != W) return fail(NTK_E_SHAPE, li + ": shared expert matrices do not have the configured sizes");
         if (form_.shared_gate) LS_TRY(upload_vector(f, p + "mlp.shared.sg", W, &M.shared_gate));
     }
     return NTK_OK;
@@ -814,6 +881,13 @@ int LayerStackModel::load(const std::string& dir, const SeqLoadOptions& opt) {
     else LS_TRY(upload_matrix(f, {"head"}, W, head_));
     if (embed_.out_f != info_.vocab || head_.out_f != info_.vocab) return fail(NTK_E_SHAPE, "embed / head do not have 'vocab' rows");
     LS_TRY(upload_norm(f, "final.norm", final_norm_));
+    if (form_.post_norm) {
+        std::vector<double> fr((size_t)(W + 1) / 2);
+        for (size_t i = 0; i < fr.size(); ++i) fr[i] = std::pow(kPositionBase, -2.0 * (double)i / W);
+        sin_freq_ = (double*)dev_alloc(fr.size() * sizeof(double));
+        if (!sin_freq_) return fail(NTK_E_NOMEM, "out of device memory");
+        nt_hip_memcpy_h2d(sin_freq_, fr.data(), fr.size() * sizeof(double));
+    }
     if (buckets_ > 0) {
         LS_TRY(upload_matrix(f, {"bigram"}, W, bigram_));
         if (bigram_.out_f != (int64_t)buckets_ + 1) return fail(NTK_E_SHAPE, "tensor 'bigram' does not have buckets + 1 rows");
@@ -895,7 +969,8 @@ int LayerStackModel::alloc_buffers() {
         if (form_.gated && L.has_mlp) max_gu2_ = std::max<int>(max_gu2_, (int)L.gff.in.out_f), max_ffn_ = std::max(max_ffn_, L.gff.ff);
         if (L.mlp_kind == kMlpMoe) {
             max_top_ = std::max(max_top_, L.mlp.top);
-            max_e_ = std::max(max_e_, L.mlp.experts);
+            max_e_ = std::max(max_e_, L.mlp.experts + L.mlp.identity);
+            max_mid_ = std::max(max_mid_, (size_t)L.mlp.top * L.mlp.routed.ff + (L.mlp.has_shared ? L.mlp.shared.ff : 0));
             max_ff2_ = std::max(max_ff2_, 2 * L.mlp.routed.ff);
             if (L.mlp.has_shared) max_sff2_ = std::max(max_sff2_, 2 * L.mlp.shared.ff);
         } else if (L.mlp_kind == kMlpDense && !form_.gated) {
@@ -919,6 +994,7 @@ int LayerStackModel::alloc_buffers() {
     if (form_.scaled)
         ok = ok && fl(&ff_, C * W) && fl(&zf_, C * std::max(max_ffn_, 1)) && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc) && fl(&rscratch_, rsc) &&
              fl(&cv_, C * std::max(max_conv_, 1)) && fl(&vfirst_, C * std::max(max_gv_, 1));
+    if (form_.post_norm) ok = ok && fl(&ff_, C * W) && fl(&zf_, C * std::max(max_ffn_, 1)) && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc) && fl(&mid_, (size_t)ntk_dense_few_rows() * max_mid_);
     if (form_.dense_parallel) ok = ok && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc);
     want_dev_ = tokens_dev_ ? tokens_dev_ + C : nullptr;   // one staging area: [tokens of a pass | wanted places], filled by ONE stream-ordered copy from pinned memory
     h_stage_ = (int*)nt_hip_malloc_host(2 * C * sizeof(int));
@@ -934,8 +1010,8 @@ int LayerStackModel::alloc_buffers() {
     for (auto& r : runs_) {
         const StackLayer& L = layers_[(size_t)r.layer];
         const size_t row = (size_t)L.cache_row();
-        if (L.att.kv_from >= 0) {
-            r.cache = runs_[(size_t)L.att.kv_from].cache;     // (such a form has no repeated span: run i is layer i)
+        if (L.kv_from() >= 0) {
+            r.cache = runs_[(size_t)L.kv_from()].cache;       // (such a form has no repeated span: run i is layer i)
         } else if (row) {
             r.cache = (float*)dev_alloc((size_t)opt_.slots * ctx * row * sizeof(float));
             if (!r.cache) return fail(NTK_E_NOMEM, "out of device memory (cache)");
@@ -964,16 +1040,17 @@ int LayerStackModel::truncate_slot(int slot, int length) {
 }
 
 // ------------------------------------------------------------------------------------------------------------------------ the step
-int LayerStackModel::run_mixer(const StackLayer& L, float* cache, int T, int pos0, bool normed_input) {
+int LayerStackModel::run_mixer(const StackLayer& L, float* cache, int T, int pos0, const float* h, bool norm_inside) {
     const LatentMixer& m = L.mix;
     const int W = info_.width, H = m.heads, qd = m.qd(), row = m.row(), hv = H * m.vdim, na = (int)m.in.out_f;
-    // one product for [query (latent) | latent + key part | gate]; decoding: the layer's first norm and the query latent's norm run inside the products
-    // (normed_input: h1_ holds the normed stream already -- the seam in front of the mixer wrote it)
+    // one product for [query (latent) | latent + key part | gate] of the mixer's input h; norm_inside (few rows): h is the stream, the layer's first norm runs
+    // inside the product; the query latent's norm runs inside its own when the rows are few
     const bool few = T <= ntk_dense_few_rows();
     ntk_dense_desc d{};
-    d.Y = a_; d.ldy = na; d.X = few && !normed_input ? x_ : h1_; d.ldx = W; d.W = m.in.ptr; d.wdtype = m.in.dtype; d.G = 1; d.row_div = 1; d.T = T; d.N = na; d.K = W;
-    if (few && !normed_input) { d.norm_w = L.norm1.w; d.norm_eps = eps_; d.norm_offset = norm_offset_; }
-    LS_TRY(ntk_dense(&d, stream_));
+    d.Y = a_; d.ldy = na; d.X = h; d.ldx = W; d.W = m.in.ptr; d.wdtype = m.in.dtype; d.G = 1; d.row_div = 1; d.T = T; d.N = na; d.K = W;
+    if (norm_inside) { d.norm_w = L.norm1.w; d.norm_eps = eps_; d.norm_offset = norm_offset_; }
+    LS_TRY(first_product(d));
+    d.add_y = nullptr;
     float* q = a_;
     int ldq = na;
     if (m.q_rank) {
@@ -985,9 +1062,12 @@ int LayerStackModel::run_mixer(const StackLayer& L, float* cache, int T, int pos
         ldq = H * qd;
     }
     ntk_rotary rot{m.rot_freq, m.rot_mag, m.rot_dims, m.rot_layout};
-    LS_TRY(ntk_latent_prepare(cache, row, a_ + m.kv_off, na, m.kv_norm, eps_, m.kv_rank, m.rot_dim, q, ldq, H, qd, &rot, pos0, T, stream_));
+    const bool own = m.kv_from < 0;                       // (else: the rows another layer wrote for these tokens earlier in the pass)
+    const bool beside = own && m.rot_dim == 0 && T <= kSharedRows;      // nothing rotated, few tokens: the cache rows are written beside the queries' fold
+    if (own && !beside) LS_TRY(ntk_latent_prepare(cache, row, a_ + m.kv_off, na, m.kv_norm, eps_, m.kv_rank, m.rot_dim, q, ldq, H, qd, &rot, pos0, T, stream_));
     if (T <= kSharedRows) {
-        LS_TRY(ntk_latent_fold_query(qf_, q, ldq, m.uk.ptr, m.uk.dtype, T, H, m.dim, m.rot_dim, m.kv_rank, stream_));
+        if (beside) LS_TRY(ntk_latent_fold_query_prepare(qf_, q, ldq, m.uk.ptr, m.uk.dtype, T, H, m.dim, m.kv_rank, cache, row, a_ + m.kv_off, na, m.kv_norm, eps_, pos0, stream_));
+        else LS_TRY(ntk_latent_fold_query(qf_, q, ldq, m.uk.ptr, m.uk.dtype, T, H, m.dim, m.rot_dim, m.kv_rank, stream_));
         LS_TRY(ntk_latent_attention(lat_, H * m.kv_rank, qf_, H * row, nullptr, 0, nullptr, 0, cache, row, m.kv_rank, m.rot_dim, H, m.dim, m.vdim, 1, pos0, T, 0,
                                     m.window, m.scale, scratch_, stream_));
         LS_TRY(ntk_latent_unfold_value_ex(att_, hv, lat_, m.uv.ptr, m.uv.dtype, a_ + m.g_off, na, m.head_gate ? 1 : 0, T, H, m.vdim, m.kv_rank, stream_));
@@ -1005,10 +1085,12 @@ int LayerStackModel::run_mixer(const StackLayer& L, float* cache, int T, int pos
 }
 
 // the window mixer: one product for [q | k | v], rotation and cache rows, attention over the window, output projection -> mix_
-int LayerStackModel::run_window(const StackLayer& L, float* cache, int T, int pos0) {
+int LayerStackModel::run_window(const StackLayer& L, const float* h, float* cache, int T, int pos0) {
     const WindowMixer& m = L.att;
     const int W = info_.width, na = (int)m.in.out_f, hv = m.heads * m.vdim;
-    LS_TRY(ntk_dense_linear(a_, na, h1_, W, m.in.ptr, m.in.dtype, T, na, W, 0, stream_));
+    ntk_dense_desc d{};
+    d.Y = a_; d.ldy = na; d.X = h; d.ldx = W; d.W = m.in.ptr; d.wdtype = m.in.dtype; d.G = 1; d.row_div = 1; d.T = T; d.N = na; d.K = W;
+    LS_TRY(first_product(d));
     LS_TRY(window_heads(m, cache, att_, hv, T, pos0));
     return ntk_dense_linear(mix_, W, att_, hv, m.o.ptr, m.o.dtype, T, W, hv, 0, stream_);
 }
@@ -1019,10 +1101,11 @@ int LayerStackModel::window_heads(const WindowMixer& m, float* cache, float* out
     ntk_rotary rot{m.rot_freq, m.rot_mag, m.rot_dims, form_.rot_halves ? NTK_ROT_HALVES : NTK_ROT_NEIGHBOURS};
     ntk_window_prepare_desc pd{};
     pd.q = a_; pd.ldq = na;
-    pd.H = m.heads; pd.G = m.kv_heads; pd.maps = m.maps; pd.dn = m.dim; pd.dv = m.vdim; pd.rot = &rot; pd.temp_every = 1.0; pd.pos0 = pos0; pd.T = T;
-    pd.q_norm = m.q_norm; pd.norm_eps = eps_;
+    pd.H = m.heads; pd.G = m.kv_heads; pd.maps = m.maps; pd.dn = m.dim; pd.dv = m.vdim; pd.rot = &rot; pd.pos0 = pos0; pd.T = T;
+    pd.q_norm = m.q_norm; pd.norm_eps = eps_; pd.head_norm = m.head_norm ? 1 : 0;
+    pd.temp_coef = m.temp_coef; pd.temp_every = m.temp_every;
     if (m.kv_from < 0) {       // (else: the rows another layer wrote for these tokens earlier in the pass)
-        pd.cache = cache; pd.row = m.row(); pd.k = a_ + m.k_off; pd.ldk = na; pd.v = a_ + m.v_off; pd.ldv = na; pd.k_norm = m.k_norm;
+        pd.cache = cache; pd.row = m.row(); pd.k = a_ + m.k_off; pd.ldk = na; pd.v = a_ + (m.raw_key_values ? m.k_off : m.v_off); pd.ldv = na; pd.k_norm = m.k_norm;
     }
     if (m.v_mix && m.v_source) { pd.v_keep = vfirst_; pd.ld_keep = m.kv_heads * m.vdim; }                 // the first blending layer keeps its values of this pass's tokens
     else if (m.v_mix) { pd.v_other = vfirst_; pd.ld_other = m.kv_heads * m.vdim; pd.v_blend = m.v_blend; }    // the later ones blend with them
@@ -1033,6 +1116,7 @@ int LayerStackModel::window_heads(const WindowMixer& m, float* cache, float* out
     d.sub_norm = m.maps == 2 ? 1 : 0; d.eps = eps_; d.out_scale = m.maps == 2 ? 1.0f - m.diff : 1.0f;
     d.scratch = wscratch_;
     d.mask_mode = m.mask_mode; d.softcap = m.softcap; d.sink = m.sink ? 1 : 0; d.keep_first = m.keep_first; d.sinks = m.sinks;
+    d.slopes = m.slopes;
     if (m.gated) { d.gate = a_ + m.g_off; d.ldg = na; d.head_gate = m.head_gate ? 1 : 0; }     // the gate rides in the launch that writes the heads' results
     return ntk_window_attention(&d, stream_);
 }
@@ -1079,16 +1163,21 @@ int LayerStackModel::run_lightning(const StackLayer& L, float* state, int T, int
 int LayerStackModel::run_experts(float glu_alpha, float glu_up_offset, const GatedExperts& ex, const float* h, float* gu, float* act, float* out, int rows, const int* offsets, const int* order, int top) {
     const int W = info_.width;
     ntk_dense_desc d{};
-    d.Y = gu; d.ldy = 2 * ex.ff; d.X = h; d.ldx = W; d.W = ex.gate_up.ptr; d.wstride = ex.gate_up.stride(); d.wdtype = ex.gate_up.dtype;
-    d.offsets = offsets; d.G = ex.gate_up.count; d.rows = order; d.row_div = top; d.T = rows; d.N = 2 * ex.ff; d.K = W; d.accumulate = 0;
-    if (rows <= ntk_dense_few_rows()) {   // decoding: the activation inside the product's launch
+    d.Y = gu; d.ldy = ex.in_rows(); d.X = h; d.ldx = W; d.W = ex.gate_up.ptr; d.wstride = ex.gate_up.stride(); d.wdtype = ex.gate_up.dtype;
+    d.offsets = offsets; d.G = ex.gate_up.count; d.rows = order; d.row_div = top; d.T = rows; d.N = ex.in_rows(); d.K = W; d.accumulate = 0;
+    if (ex.plain) {                       // the activation inside the product, whatever its form
+        d.Y = act; d.act = NTK_ACT_RELU2;
+        LS_TRY(first_product(d));
+        d.act = NTK_ACT_NONE;
+    } else if (rows <= ntk_dense_few_rows()) {   // decoding: the activation inside the product's launch
         d.Y = act; d.ldy = ex.ff; d.glu_ff = ex.ff; d.glu_limit = ex.limit; d.glu_alpha = glu_alpha; d.glu_up_offset = glu_up_offset;
-        LS_TRY(ntk_dense(&d, stream_));
+        LS_TRY(first_product(d));
         d.glu_ff = 0;
     } else {
         LS_TRY(ntk_dense(&d, stream_));
         LS_TRY(ntk_glu(act, gu, rows, ex.ff, ex.limit, glu_alpha, glu_up_offset, stream_));
     }
+    d.add_y = nullptr;
     d.Y = out; d.ldy = W; d.X = act; d.ldx = ex.ff; d.W = ex.down.ptr; d.wstride = ex.down.stride(); d.wdtype = ex.down.dtype;
     d.rows = nullptr; d.row_div = 1; d.N = W; d.K = ex.ff;
     return ntk_dense(&d, stream_);
@@ -1096,16 +1185,29 @@ int LayerStackModel::run_experts(float glu_alpha, float glu_up_offset, const Gat
 
 // router, grouping, the experts' products; then either straight into the stream together with the mixer's output (parallel form) or as a sum of its own
 // in ff_ (sequential form: it is normed before it joins the stream)
-int LayerStackModel::run_moe(const StackLayer& L, int T, bool into_stream) {
+int LayerStackModel::run_moe(const StackLayer& L, const float* h, int T, bool into_stream) {
     const MoeFeedForward& M = L.mlp;
-    const int W = info_.width;
+    const int W = info_.width, choices = M.experts + M.identity;
     float* sgate = M.has_shared && M.shared_gate ? sg_ : nullptr;
-    LS_TRY(ntk_moe_route_ex(ids_, wts_, sgate, h2_, W, M.router, sgate ? M.shared_gate : nullptr, T, W, M.experts, M.top, &M.route, stream_));
-    LS_TRY(ntk_moe_group(offsets_, order_, where_, ids_, T, M.top, M.experts, stream_));
-    LS_TRY(run_experts(M.glu_alpha, M.glu_up_offset, M.routed, h2_, gu_, act_, dn_, T * M.top, offsets_, order_, M.top));
-    if (M.has_shared) LS_TRY(run_experts(M.glu_alpha, M.glu_up_offset, M.shared, h2_, sgu_, sact_, sdn_, T, nullptr, nullptr, 1));
+    ntk_route_desc route = M.route;
+    if (form_.post_norm && owed_.y) {      // what the stream is still owed joins it in the router's launch
+        route.add_y = owed_.y; route.ld_add = W; route.add_w = owed_.nb.w; route.add_eps = eps_;
+        owed_.y = nullptr;
+    }
+    LS_TRY(ntk_moe_route_ex(ids_, wts_, sgate, h, W, M.router, sgate ? M.shared_gate : nullptr, T, W, choices, M.top, &route, stream_));
+    const size_t mid = (size_t)M.top * M.routed.ff + (M.has_shared ? M.shared.ff : 0);
+    if (M.routed.plain && T <= ntk_dense_few_rows() && mid <= NTK_MOE_FEW_MID && W <= NTK_MOE_FEW_MID && !into_stream) {     // decoding: two launches for all of a token's units
+        ntk_moe_few_desc d{};
+        d.out = ff_; d.ldo = W; d.h = h; d.ldh = W; d.ids = ids_; d.wts = wts_; d.top = M.top; d.experts = M.experts; d.up = M.routed.gate_up.ptr; d.down = M.routed.down.ptr; d.ff = M.routed.ff;
+        if (M.has_shared) { d.shared_up = M.shared.gate_up.ptr; d.shared_down = M.shared.down.ptr; d.shared_ff = M.shared.ff; d.sgate = sgate; }
+        d.wdtype = M.routed.down.dtype; d.act = NTK_ACT_RELU2; d.mid = mid_; d.T = T; d.n = W;
+        return ntk_moe_few(&d, stream_);
+    }
+    LS_TRY(ntk_moe_group(offsets_, order_, where_, ids_, T, M.top, choices, stream_));     // (identity experts come last: rows behind offsets_[experts], which no product visits)
+    LS_TRY(run_experts(M.glu_alpha, M.glu_up_offset, M.routed, h, gu_, act_, dn_, T * M.top, offsets_, order_, M.top));
+    if (M.has_shared) LS_TRY(run_experts(M.glu_alpha, M.glu_up_offset, M.shared, h, sgu_, sact_, sdn_, T, nullptr, nullptr, 1));
     if (into_stream) return ntk_moe_combine(x_, mix_, dn_, where_, wts_, M.has_shared ? sdn_ : nullptr, sgate, T, M.top, W, stream_);
-    return ntk_moe_sum(ff_, dn_, where_, wts_, M.has_shared ? sdn_ : nullptr, sgate, T, M.top, W, stream_);
+    return ntk_moe_sum_ex(ff_, dn_, where_, M.identity ? ids_ : nullptr, M.experts, h, W, wts_, M.has_shared ? sdn_ : nullptr, sgate, T, M.top, W, stream_);
 }
 
 // up, the polynomial activation over every token's row of ff values, down -> ff_ (the activation runs in place in the up product's buffer)
@@ -1117,9 +1219,9 @@ int LayerStackModel::run_dense_ff(const StackLayer& L, int T) {
     return ntk_dense_linear(ff_, W, zf_, D.ff, D.down.ptr, D.down.dtype, T, W, D.ff, 0, stream_);
 }
 
-// the dense clipped gated unit (the experts' unit with one member): gate and up in one product (decoding: the activation inside its launch), down -> ff_
-int LayerStackModel::run_clipped_ff(const StackLayer& L, int T) {
-    return run_experts(kGluAlpha, 1.0f, L.cff, h2_, gu2_, zf_, ff_, T, nullptr, nullptr, 1);
+// the dense gated unit (the experts' unit with one member, clipped or plain): gate and up in one product (decoding: the activation inside its launch), down -> ff_
+int LayerStackModel::run_unit_ff(const StackLayer& L, const float* h, int T) {
+    return run_experts(form_.clipped_glu ? kGluAlpha : 1.0f, form_.clipped_glu ? 1.0f : 0.0f, L.cff, h, gu2_, zf_, ff_, T, nullptr, nullptr, 1);
 }
 
 // the delta rule with per-head gates: one product for [q | k | v | gate | beta | decay], the short convolutions of q, k and v (+ silu) with their carried
@@ -1157,14 +1259,42 @@ int LayerStackModel::rms_seam(const NormW& nw, float* out, int T) {
 
 int LayerStackModel::scaled_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0) {
     LS_TRY(rms_seam(L.norm1, h1_, T));
-    if (L.mixer == kMixWindow) LS_TRY(run_window(L, run.cache + (size_t)slot * opt_.max_context * L.att.row(), T, pos0));
-    else if (L.mixer == kMixLatent) LS_TRY(run_mixer(L, run.cache + (size_t)slot * opt_.max_context * L.mix.row(), T, pos0, true));
+    if (L.mixer == kMixWindow) LS_TRY(run_window(L, h1_, run.cache + (size_t)slot * opt_.max_context * L.att.row(), T, pos0));
+    else if (L.mixer == kMixLatent) LS_TRY(run_mixer(L, run.cache + (size_t)slot * opt_.max_context * L.mix.row(), T, pos0, h1_));
     else LS_TRY(run_gated_delta(L, run.state + (size_t)slot * L.gdl.state_floats(), T, pos0));
     owed_ = Owed{mix_, L.norm1b};
     if (!L.has_mlp) return NTK_OK;
     LS_TRY(rms_seam(L.norm2, h2_, T));
-    LS_TRY(run_clipped_ff(L, T));
+    LS_TRY(run_unit_ff(L, h2_, T));
     owed_ = Owed{ff_, L.norm2b};
+    return NTK_OK;
+}
+
+// The first product of a sublayer.  In the post-norm form it reads the stream itself: with few rows, what the stream is still owed joins it inside this launch, which
+// leaves the new stream in the other buffer (its workgroups all read the old one).
+int LayerStackModel::first_product(ntk_dense_desc& d) {
+    if (!form_.post_norm || !owed_.y || d.X != x_) return ntk_dense(&d, stream_);
+    const int W = info_.width;
+    d.add_y = owed_.y; d.ld_add = W; d.add_w = owed_.nb.w; d.add_eps = eps_; d.add_mult = residual_mult_; d.x_out = x0_; d.ldxo = W;
+    LS_TRY(ntk_dense(&d, stream_));
+    std::swap(x_, x0_);
+    owed_.y = nullptr;
+    return NTK_OK;
+}
+
+// A layer of the post-norm form: a sublayer reads the stream itself, and its result joins the stream through a norm of its own (decoding: on the way into the next
+// sublayer's first product or router; prompts: in a launch between them).
+int LayerStackModel::post_norm_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0) {
+    const bool few = T <= ntk_dense_few_rows();
+    if (!few) LS_TRY(settle(T));
+    if (L.mixer == kMixWindow) LS_TRY(run_window(L, x_, run.cache + (size_t)slot * opt_.max_context * L.att.row(), T, pos0));
+    else LS_TRY(run_mixer(L, run.cache + (size_t)slot * opt_.max_context * L.mix.row(), T, pos0, x_));
+    owed_ = Owed{mix_, L.norm1};
+    if (!L.has_mlp) return NTK_OK;
+    if (!few && L.mlp_kind != kMlpMoe) LS_TRY(settle(T));      // (the router's launch does it for any number of tokens)
+    if (L.mlp_kind == kMlpMoe) LS_TRY(run_moe(L, x_, T, false));
+    else LS_TRY(run_unit_ff(L, x_, T));
+    owed_ = Owed{ff_, L.norm2};
     return NTK_OK;
 }
 
@@ -1280,7 +1410,7 @@ int LayerStackModel::norm_conv(const NormW& nw, const float* canon, float* conv_
 int LayerStackModel::settle(int T) {
     if (!owed_.y) return NTK_OK;
     const int W = info_.width;
-    const int st = form_.scaled ? ntk_rms_seam(nullptr, 0, x_, W, owed_.y, W, owed_.nb.w, residual_mult_, nullptr, T, W, eps_, stream_)
+    const int st = form_.scaled || form_.post_norm ? ntk_rms_seam(nullptr, 0, x_, W, owed_.y, W, owed_.nb.w, residual_mult_, nullptr, T, W, eps_, stream_)
                                 : ntk_layernorm(x_, W, owed_.y, W, owed_.nb.w, owed_.nb.b, T, W, eps_, 1, stream_);
     owed_.y = nullptr;
     return st;
@@ -1290,12 +1420,12 @@ int LayerStackModel::sequential_layer(const Run& run, const StackLayer& L, int s
     const int W = info_.width;
     float* conv = run.conv ? run.conv + (size_t)slot * 2 * (taps_ - 1) * W : nullptr;
     LS_TRY(norm_conv(L.norm1, L.canon1, conv, h1_, T, pos0));
-    if (L.mixer == kMixWindow) LS_TRY(run_window(L, run.cache + (size_t)slot * opt_.max_context * L.att.row(), T, pos0));
+    if (L.mixer == kMixWindow) LS_TRY(run_window(L, h1_, run.cache + (size_t)slot * opt_.max_context * L.att.row(), T, pos0));
     else LS_TRY(run_lightning(L, run.state + (size_t)slot * L.lin.state_floats(), T, pos0));
     owed_ = Owed{mix_, L.norm1b};
     if (!L.has_mlp) return NTK_OK;
     LS_TRY(norm_conv(L.norm2, L.canon2, conv ? conv + (size_t)(taps_ - 1) * W : nullptr, h2_, T, pos0));
-    if (L.mlp_kind == kMlpMoe) LS_TRY(run_moe(L, T, false));
+    if (L.mlp_kind == kMlpMoe) LS_TRY(run_moe(L, h2_, T, false));
     else LS_TRY(run_dense_ff(L, T));
     owed_ = Owed{ff_, L.norm2b};
     return NTK_OK;
@@ -1309,8 +1439,9 @@ int LayerStackModel::parallel_layer(const Run& run, const StackLayer& L, int slo
         LS_TRY(ntk_rmsnorm_offset(h2_, L.norm2.w, nullptr, nullptr, W, x_, W, T, W, eps_, 1.0f, stream_));
     }
     float* cache = run.cache + (size_t)slot * opt_.max_context * L.mix.row();
-    LS_TRY(run_mixer(L, cache, T, pos0));
-    if (L.has_mlp) return run_moe(L, T, true);
+    const bool few = T <= ntk_dense_few_rows();
+    LS_TRY(run_mixer(L, cache, T, pos0, few ? x_ : h1_, few));
+    if (L.has_mlp) return run_moe(L, h2_, T, true);
     return ntk_residual_add(x_, mix_, nullptr, T * W, stream_);
 }
 
@@ -1324,6 +1455,8 @@ int LayerStackModel::portion(int slot, const int* tokens_dev, int prev_token, in
                                    embed_norm_.alpha, stream_));
         const NormW& n1 = layers_[(size_t)runs_[0].layer].norm1;
         LS_TRY(ntk_dyt(h1_, W, x_, W, n1.w, n1.b, n1.alpha, T, W, stream_));
+    } else if (form_.post_norm) {
+        LS_TRY(ntk_embed_sinusoid(x_, embed_.ptr, embed_.dtype, tokens_dev, T, info_.vocab, W, embed_scale_, sin_freq_, pos0, stream_));
     } else if (buckets_ > 0) {
         LS_TRY(ntk_embed_bigram(x_, embed_.ptr, bigram_.ptr, embed_.dtype, tokens_dev, prev_token, pos0, T, info_.vocab, W, embed_scale_, buckets_, mul_prev_, mul_cur_, stream_));
     } else
@@ -1347,6 +1480,9 @@ int LayerStackModel::portion(int slot, const int* tokens_dev, int prev_token, in
         } else if (form_.sequential) {
             LS_TRY(sequential_layer(run, L, slot, T, pos0));
             if (r + 1 == runs_.size() || (capture_ && capture_buf_)) LS_TRY(settle(T));
+        } else if (form_.post_norm) {
+            LS_TRY(post_norm_layer(run, L, slot, T, pos0));
+            if ((r + 1 == runs_.size() && !(T == 1 && n_want == 1)) || (capture_ && capture_buf_)) LS_TRY(settle(T));
         } else if (form_.dense_parallel) {
             LS_TRY(dense_parallel_layer(run, L, slot, T, pos0));
         } else {
@@ -1362,7 +1498,8 @@ int LayerStackModel::portion(int slot, const int* tokens_dev, int prev_token, in
         ntk_dense_desc d{};
         d.Y = logits_out; d.ldy = info_.vocab; d.X = rows; d.ldx = W; d.W = head_.ptr; d.wdtype = head_.dtype; d.G = 1; d.row_div = 1; d.T = n_want;
         d.N = info_.vocab; d.K = W;
-        if (form_.gated) { LS_TRY(ntk_dyt(hn_, W, rows, W, final_norm_.w, final_norm_.b, final_norm_.alpha, n_want, W, stream_)); d.X = hn_; }
+        if (form_.post_norm && owed_.y) { LS_TRY(rms_seam(final_norm_, hn_, T)); d.X = hn_; }      // a single decoded token: what it is still owed and the output norm in one launch
+        else if (form_.gated) { LS_TRY(ntk_dyt(hn_, W, rows, W, final_norm_.w, final_norm_.b, final_norm_.alpha, n_want, W, stream_)); d.X = hn_; }
         else if (final_norm_.b) { LS_TRY(ntk_layernorm(hn_, W, rows, W, final_norm_.w, final_norm_.b, n_want, W, eps_, 0, stream_)); d.X = hn_; }
         else if (n_want <= ntk_dense_few_rows()) { d.norm_w = final_norm_.w; d.norm_eps = eps_; d.norm_offset = norm_offset_; }   // the output norm inside the head's launch
         else { LS_TRY(ntk_rmsnorm_offset(hn_, final_norm_.w, nullptr, nullptr, W, rows, W, n_want, W, eps_, norm_offset_, stream_)); d.X = hn_; }

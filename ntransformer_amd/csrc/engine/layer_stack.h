@@ -16,6 +16,8 @@
 //   scaled       x += m * norm1b(mixer(norm1 x)), then x += m * norm2b(ff(norm2 x)): RMS norms with a plain weight before and after every sublayer, one
 //                fixed factor m on everything that joins the stream, scaled embedding, the embedding table as the head, capped logits
 //                                                                                                                           -- "Fifotar"
+//   post_norm    x += norm1(mixer(x)), then x += norm2(ff(x)): no norm in front of a sublayer, RMS norms with a plain weight on their results only, a
+//                sinusoidal position vector added to the embedding                                                          -- "Gibevik"
 //
 // Mechanisms are parsed into parameter structs and run by the operators of include/ntk_layers.h, so another family can list them in another order
 // or with other constants:
@@ -34,10 +36,14 @@
 //                 in the dense parallel form "attention" is grouped-query attention over a sliding window beside which a sequence's first positions stay
 //                 visible, with queries and keys normed over their whole projection, half-split rotation with blended frequencies, a learned sink and one gate
 //                 per head, and optionally the keys and values of an EARLIER layer instead of its own (the same WindowMixer and kernels);
+//                 in the post-norm form "attention" is causal grouped-query attention whose values are its keys as projected, with queries and keys normed per
+//                 head, a query temperature, a bias falling with the distance and an elementwise gate, and "latent_attention" has no rotated part, a query from one
+//                 matrix, a gate per head and optionally the latents of an earlier layer (the same WindowMixer, LatentMixer and kernels);
 //   feed-forward  kind "moe": routed gated experts + an optional shared expert (MoeFeedForward: softmax or sigmoid scores, optional expert groups,
 //                 clipped or plain gated units); kind "dense": up, polynomial activation with unit-norm terms, down (DenseFeedForward), or in the
 //                 gated form a gated unit with the tanh form of gelu (GatedFeedForward), in the scaled form the clipped gated unit of the experts as one
-//                 dense unit, in the dense parallel form the plain one (GatedExperts with one member).
+//                 dense unit, in the dense parallel and the post-norm form the plain one (GatedExperts with one member).  In the post-norm form the experts are plain units
+//                 (squared relu between two matrices), chosen with a correction added to their scores, some of them the identity.
 // What a sequence holds per layer run: cache rows per position (attention kinds; none where a layer reads another one's), a recurrent state (lightning, gla, delta
 // rules), the convolutions' last inputs; and per slot its token ids where the embedding reads the token before.
 #pragma once
@@ -65,6 +71,7 @@ struct LatentMixer {
     float rot_mag = 1.0f;
     int rot_layout = NTK_ROT_NEIGHBOURS;
     bool head_gate = false;           // the output gate is one number per head (else one per head and value entry)
+    int kv_from = -1;                 // >= 0: no latents of its own, it reads the cache rows of that layer
     double* rot_freq = nullptr;       // device [rot_dims / 2]
     DenseW in;                        // rows [query or query latent | kv_rank + rot_dim | gate] of one product over the normed input
     int q_off = 0, kv_off = 0, g_off = 0;
@@ -87,9 +94,14 @@ struct WindowMixer {                  // grouped-query attention, sliding window
     int keep_first = 0;               // positions that stay visible beside a sliding window
     bool sink = false;                // one more exp(0) in every softmax's denominator
     float* sinks = nullptr;           // ... or exp(sinks[h]), F32 [heads]
+    float* slopes = nullptr;          // F32 [heads]: slopes[h] * distance comes off the scaled score
+    bool head_norm = false;           // q_norm and k_norm are [dim], every head normed on its own, ahead of the temperature
+    float temp_coef = 0.0f;           // query temperature 1 + coef ln(floor((p + 1) / every) + 1)
+    double temp_every = 1.0;
+    bool raw_key_values = false;      // the values are the keys as projected (no rows of v in `in`)
     bool gated = false;               // sigmoid gate on the joined heads (its rows sit behind v in `in`), elementwise or one number per head
     bool head_gate = false;
-    float *q_norm = nullptr, *k_norm = nullptr;   // F32 [heads * dim], [kv_heads * dim]: RMS norm over the whole projection, ahead of the rotation
+    float *q_norm = nullptr, *k_norm = nullptr;   // F32 [heads * dim], [kv_heads * dim]: RMS norm over the whole projection, ahead of the rotation (or see head_norm)
     float rot_mag = 1.0f;
     int kv_from = -1;                 // >= 0: this layer has no keys and values of its own, it reads the cache rows of that layer
     bool v_mix = false, v_source = false;   // values blended with those of the first such layer (v_source: this IS that layer, it only keeps them)
@@ -172,12 +184,16 @@ struct GatedFeedForward {             // down(gelu_tanh(gate h) * (up h)), its r
 
 struct GatedExperts {                 // `count` experts of the same shape, stacked: gate rows then up rows, and the down matrices
     int ff = 0;
+    bool plain = false;               // no gate: up rows only, squared relu
+    int in_rows() const { return plain ? ff : 2 * ff; }
     float limit = 0.0f;               // clamp of the gate (from above) and the up value (both sides); INFINITY: none
     DenseW gate_up, down;
 };
 
 struct MoeFeedForward {
-    int experts = 0, top = 0;
+    int experts = 0, top = 0;         // experts with matrices; the router's choices are experts + identity
+    int identity = 0;                 // the last choices give the input itself
+    float* correction = nullptr;      // F32 [experts + identity], in route.correction: joins the scores when experts are chosen
     ntk_route_desc route{};           // score function, expert groups, renormalisation, scale of the weights
     float glu_alpha = 1.0f, glu_up_offset = 0.0f;   // act(g) = g * sigmoid(alpha g), multiplied by (up + offset)
     float* router = nullptr;          // F32 [experts][width]
@@ -219,6 +235,7 @@ struct StackLayer {
     bool has_mlp = false;
     MoeFeedForward mlp;
     DenseFeedForward ffn;
+    int kv_from() const { return mixer == kMixWindow ? att.kv_from : mixer == kMixLatent ? mix.kv_from : -1; }
     int cache_row() const { return mixer == kMixLatent ? mix.row() : mixer == kMixWindow ? att.row() : mixer == kMixParallel ? par.left.row() : 0; }
     size_t state_floats() const {
         return mixer == kMixLightning ? lin.state_floats() : mixer == kMixGla ? gla.state_floats() : mixer == kMixParallel ? par.right.state_floats() :
@@ -232,20 +249,27 @@ struct StackForm {
     bool gated = false;               // ...
     bool scaled = false;              // ... (none of the three: the parallel form)
     bool dense_parallel = false;      // the parallel form with plain norm weights, window attention and one dense gated unit
+    bool post_norm = false;           // ...
     bool blended_rotation = false;    // an attention layer's rotary scaling: a ramp over the pair index, with a magnitude (else by wavelength)
     bool learned_sinks = false;       // an attention layer's softmax has a learned sink per head
     bool attention_head_gate = false; // its output gate is one number per head
     bool whole_qk_norm = false;       // its queries and keys are normed over the whole projection
+    bool head_qk_norm = false;        // ... or per head with one shared weight
+    bool raw_key_values = false;      // its values are its keys as projected
+    bool distance_slopes = false;     // its scores fall with the distance, 2^(-8 (h + 1) / heads) per position in head h
     // the scaled form's mechanisms: what its design fixes about them
     bool mask_chunks = false;         // an attention layer's mask.size is a chunk size (else a sliding window)
     bool attention_sink = false;      // its softmax has a sink
     bool attention_gate = false;      // ... and an elementwise output gate
     bool rot_halves = false;          // rotated entries are paired half against half (else neighbours)
     bool latent_head_gate = false;    // latent attention's output gate is one number per head
+    bool latent_plain = false;        // it has neither a rotated part nor a query latent
     bool loop_projection = true;      // the repeated span is entered through 'loop.in' over [stream ; embedding]
     int router_score = 0;             // 0 softmax, 1 sigmoid
     bool router_renorm = true;
     bool clipped_glu = true;          // experts: clipped gated unit with slope kGluAlpha and up + 1; else silu(gate) * up
+    bool plain_experts = false;       // experts without a gate: squared relu
+    bool router_correction = false;   // experts are chosen by score + a learned correction
     bool shared_gate = true;          // the shared expert sits behind a per-token sigmoid gate
     int group_top = 2;                // a group's score: the sum of this many of its largest scores
 };
@@ -287,7 +311,8 @@ private:
     int run_gated_ff(const StackLayer& L, int T);
     int parse_gated_delta(const Json& L, GatedDeltaMixer& m);
     int run_gated_delta(const StackLayer& L, float* state, int T, int pos0);
-    int run_clipped_ff(const StackLayer& L, int T);
+    int run_unit_ff(const StackLayer& L, const float* h, int T);
+    int post_norm_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0);
     int rms_seam(const NormW& nw, float* out, int T);
     int scaled_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0);
     int gated_layer(size_t r, const StackLayer& L, int slot, int T, int pos0);
@@ -301,20 +326,21 @@ private:
     int alloc_buffers();
     void* dev_alloc(size_t bytes);
     int portion(int slot, const int* tokens_dev, int prev_token, int T, int pos0, const int* want_dev, int n_want, float* logits_out);
-    int run_mixer(const StackLayer& L, float* cache, int T, int pos0, bool normed_input = false);
-    int run_window(const StackLayer& L, float* cache, int T, int pos0);
+    int run_mixer(const StackLayer& L, float* cache, int T, int pos0, const float* h, bool norm_inside = false);
+    int run_window(const StackLayer& L, const float* h, float* cache, int T, int pos0);
     int window_heads(const WindowMixer& m, float* cache, float* out, int ldo, int T, int pos0);
     int dense_parallel_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0);
     int run_lightning(const StackLayer& L, float* state, int T, int pos0);
-    int run_moe(const StackLayer& L, int T, bool into_stream);
+    int run_moe(const StackLayer& L, const float* h, int T, bool into_stream);
     int run_dense_ff(const StackLayer& L, int T);
     int run_experts(float glu_alpha, float glu_up_offset, const GatedExperts& ex, const float* h, float* gu, float* act, float* out, int rows, const int* offsets, const int* order, int top);
     int norm_conv(const NormW& nw, const float* canon, float* conv_state, float* out, int T, int pos0);
     int settle(int T);
+    int first_product(ntk_dense_desc& d);
     int sequential_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0);
     int parallel_layer(const Run& run, const StackLayer& L, int slot, int T, int pos0);
 
-    struct Owed { const float* y = nullptr; NormW nb; };   // sequential form: a sublayer's output that its norm has yet to add to the stream
+    struct Owed { const float* y = nullptr; NormW nb; };   // sequential, scaled and post-norm form: a sublayer's output that its norm has yet to add to the stream
     Owed owed_;
     StackForm form_;
     SeqModelInfo info_;
@@ -325,6 +351,7 @@ private:
     int taps_ = 1;                    // the input convolutions' taps (sequential form)
     float embed_scale_ = 1.0f, logit_scale_ = 1.0f;
     float residual_mult_ = 1.0f, logit_softcap_ = 0.0f;   // scaled form
+    double* sin_freq_ = nullptr;      // device [(width + 1) / 2]: the position vector's frequencies (post-norm form)
     float norm_offset_ = 1.0f;        // what is added to an RMS norm's stored weight: 1 where weights are stored around zero, 0 where plain
     bool has_state_ = false;          // some layer carries a recurrent state or convolution inputs: a slot can only be cut back to its start
     std::vector<StackLayer> layers_;
@@ -348,7 +375,8 @@ private:
     float *x_ = nullptr, *x0_ = nullptr, *cat_ = nullptr, *h1_ = nullptr, *h2_ = nullptr, *a_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *qf_ = nullptr, *lat_ = nullptr,
           *att_ = nullptr, *kx_ = nullptr, *vx_ = nullptr, *mix_ = nullptr, *wts_ = nullptr, *sg_ = nullptr, *gu_ = nullptr, *act_ = nullptr, *dn_ = nullptr,
           *sgu_ = nullptr, *sact_ = nullptr, *sdn_ = nullptr, *scratch_ = nullptr, *xw_ = nullptr, *hn_ = nullptr, *hist_ = nullptr, *ff_ = nullptr, *zf_ = nullptr, *wscratch_ = nullptr, *lscratch_ = nullptr,
-          *results_ = nullptr, *zq_ = nullptr, *gu2_ = nullptr, *rscratch_ = nullptr, *cv_ = nullptr, *vfirst_ = nullptr;   // gated form: the layer results of the pass [runs + 1][chunk][width], decay pre-activations, [gate | up | residual gate]
+          *results_ = nullptr, *zq_ = nullptr, *gu2_ = nullptr, *rscratch_ = nullptr, *cv_ = nullptr, *vfirst_ = nullptr, *mid_ = nullptr;   // gated form: the layer results of the pass [runs + 1][chunk][width], decay pre-activations, [gate | up | residual gate]
+    size_t max_mid_ = 0;              // (post-norm form: the experts' activations of a token side by side)
     int max_rec_ = 0, max_gu2_ = 0, max_conv_ = 0, max_gv_ = 0;   // (scaled form: convolution channels, key heads x value size of the blending attention layers)
     int *ids_ = nullptr, *offsets_ = nullptr, *order_ = nullptr, *where_ = nullptr, *tokens_dev_ = nullptr, *want_dev_ = nullptr;
     int* h_stage_ = nullptr;          // pinned: tokens and wanted places of the pass being launched

@@ -392,9 +392,21 @@ __global__ __launch_bounds__(256) void latent_attention_merge_kernel(float* out,
 // ------------------------------------------------------------------------------------------------------------------- fold / unfold
 // qf[t][h][r] = sum_d q[t][h][d] W_uk[h * dn + d][r]; rotated part copied behind.  grid (R / 64, H, T): 64 columns per workgroup, the d range in
 // four parts (one per wave), added through LDS in wave order
+// kv != NULL (dr == 0): the workgroups (0, H, T) write the tokens' normed latents into the cache rows beside that
+struct FoldPrepare { float* cache; int row; const float* kv; int ldkv; const float* norm_w; float eps; int pos0; };
 template <typename WT>
-__global__ __launch_bounds__(256) void latent_fold_query_kernel(float* qf, const float* q, int ldq, const WT* w, int H, int dn, int dr, int R) {
+__global__ __launch_bounds__(256) void latent_fold_query_kernel(float* qf, const float* q, int ldq, const WT* w, int H, int dn, int dr, int R, const FoldPrepare p) {
     extern __shared__ float qs[];      // [dn + dr] then [4][64] partial sums
+    if ((int)blockIdx.y == H) {        // (uniform over the workgroup)
+        if (blockIdx.x > 0) return;
+        const float* src = p.kv + (long long)blockIdx.z * p.ldkv;
+        float* dst = p.cache + (long long)(p.pos0 + blockIdx.z) * p.row;
+        float ss = 0.0f;
+        for (int i = threadIdx.x; i < R; i += 256) ss = fmaf(src[i], src[i], ss);
+        const float inv = 1.0f / sqrtf(block_sum(ss, qs) / (float)R + p.eps);
+        for (int i = threadIdx.x; i < R; i += 256) dst[i] = src[i] * inv * p.norm_w[i];
+        return;
+    }
     float* part = qs + dn + dr;
     const int h = blockIdx.y, t = blockIdx.z;
     const float* qh = q + (long long)t * ldq + (long long)h * (dn + dr);
@@ -467,7 +479,9 @@ using namespace ntk;
 
 int ntk_latent_prepare(float* cache, int row, const float* kv, int ldkv, const float* norm_w, float eps, int kv_rank, int rot_dim, float* q, int ldq, int H, int qd,
                        const ntk_rotary* rot, int pos0, int T, void* stream) {
-    if (!cache || !kv || !norm_w || !rot || !rot->freq) return NTK_E_NULL;
+    static const ntk_rotary none{nullptr, 1.0f, 0, NTK_ROT_NEIGHBOURS};
+    if (!rot) rot = &none;
+    if (!cache || !kv || !norm_w || (rot->dims > 0 && !rot->freq)) return NTK_E_NULL;
     if (T < 0 || kv_rank <= 0 || rot_dim < 0 || rot->dims < 0 || (rot->dims & 1) || rot->dims > rot_dim || row < kv_rank + rot_dim || ldkv < kv_rank + rot_dim || pos0 < 0) return NTK_E_SHAPE;
     if (q && (H <= 0 || qd < rot_dim || ldq < H * qd)) return NTK_E_SHAPE;
     if (rot->layout != NTK_ROT_NEIGHBOURS && rot->layout != NTK_ROT_HALVES) return NTK_E_SHAPE;
@@ -530,16 +544,27 @@ int ntk_latent_attention(float* out, int ldo, const float* q, int ldq, const flo
     return last_launch_status();
 }
 
-int ntk_latent_fold_query(float* qf, const float* q, int ldq, const void* w_uk, int wdtype, int T, int H, int dn, int dr, int R, void* stream) {
+static int fold_query(float* qf, const float* q, int ldq, const void* w_uk, int wdtype, int T, int H, int dn, int dr, int R, const FoldPrepare& p, void* stream) {
     if (!qf || !q || !w_uk) return NTK_E_NULL;
     if (T < 0 || H <= 0 || dn <= 0 || dr < 0 || R <= 0) return NTK_E_SHAPE;
     if (T == 0) return NTK_OK;
     const size_t lds = (size_t)(dn + dr + 256) * sizeof(float);
-    const dim3 grid((R + 63) / 64, H, T);
-    if (wdtype == NTK_DT_BF16) hipLaunchKernelGGL(latent_fold_query_kernel<uint16_t>, grid, dim3(256), lds, resolve_stream(stream), qf, q, ldq, (const uint16_t*)w_uk, H, dn, dr, R);
-    else if (wdtype == NTK_DT_F32) hipLaunchKernelGGL(latent_fold_query_kernel<float>, grid, dim3(256), lds, resolve_stream(stream), qf, q, ldq, (const float*)w_uk, H, dn, dr, R);
+    const dim3 grid((R + 63) / 64, H + (p.kv ? 1 : 0), T);
+    if (wdtype == NTK_DT_BF16) hipLaunchKernelGGL(latent_fold_query_kernel<uint16_t>, grid, dim3(256), lds, resolve_stream(stream), qf, q, ldq, (const uint16_t*)w_uk, H, dn, dr, R, p);
+    else if (wdtype == NTK_DT_F32) hipLaunchKernelGGL(latent_fold_query_kernel<float>, grid, dim3(256), lds, resolve_stream(stream), qf, q, ldq, (const float*)w_uk, H, dn, dr, R, p);
     else return NTK_E_DTYPE;
     return last_launch_status();
+}
+
+int ntk_latent_fold_query(float* qf, const float* q, int ldq, const void* w_uk, int wdtype, int T, int H, int dn, int dr, int R, void* stream) {
+    return fold_query(qf, q, ldq, w_uk, wdtype, T, H, dn, dr, R, FoldPrepare{}, stream);
+}
+
+int ntk_latent_fold_query_prepare(float* qf, const float* q, int ldq, const void* w_uk, int wdtype, int T, int H, int dn, int R, float* cache, int row, const float* kv,
+                                  int ldkv, const float* norm_w, float eps, int pos0, void* stream) {
+    if (!cache || !kv || !norm_w) return NTK_E_NULL;
+    if (row < R || ldkv < R || pos0 < 0) return NTK_E_SHAPE;
+    return fold_query(qf, q, ldq, w_uk, wdtype, T, H, dn, 0, R, FoldPrepare{cache, row, kv, ldkv, norm_w, eps, pos0}, stream);
 }
 
 int ntk_latent_unfold_value(float* out, int ldo, const float* lat, const void* w_uv, int wdtype, const float* gate, int ldg, int T, int H, int dv, int R,

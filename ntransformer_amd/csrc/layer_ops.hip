@@ -42,6 +42,20 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(float* out, const TT*
     out[(long long)t * width + i] = fmaf(ok ? e : 0.0f, scale, b);
 }
 
+// a thread owns the pair (2i, 2i + 1): sin and cos of one angle, formed in double
+template <typename TT>
+__global__ __launch_bounds__(256) void embed_sinusoid_kernel(float* out, const TT* table, const int* tokens, int vocab, int width, float scale, const double* freq, int pos0) {
+    const int t = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x, tok = tokens[t];
+    if (2 * i >= width) return;
+    const bool ok = tok >= 0 && tok < vocab;
+    const TT* row = table + (long long)(ok ? tok : 0) * width;
+    float* o = out + (long long)t * width;
+    double sn, cs;
+    sincos((double)(pos0 + t) * freq[i], &sn, &cs);
+    o[2 * i] = fmaf(ok ? table_value(row, 2 * i) : 0.0f, scale, (float)sn);
+    if (2 * i + 1 < width) o[2 * i + 1] = fmaf(ok ? table_value(row, 2 * i + 1) : 0.0f, scale, (float)cs);
+}
+
 __global__ __launch_bounds__(256) void rmsnorm_offset_kernel(float* y1, const float* w1, float* y2, const float* w2, int ldy, const float* x, int ldx, int n,
                                                              float eps, float offset) {
     __shared__ float red[16];
@@ -247,6 +261,19 @@ int ntk_embed_bigram(float* out, const void* table, const void* bigram, int tdty
     else
         hipLaunchKernelGGL(embed_bigram_kernel<float>, grid, dim3(256), 0, resolve_stream(stream), out, (const float*)table, (const float*)bigram, tokens, prev, pos0,
                            vocab, width, scale, buckets, mul_prev, mul_cur);
+    return last_launch_status();
+}
+
+int ntk_embed_sinusoid(float* out, const void* table, int tdtype, const int* tokens, int T, int vocab, int width, float scale, const double* freq, int pos0, void* stream) {
+    if (!out || !table || !tokens || !freq) return NTK_E_NULL;
+    if (tdtype != NTK_DT_BF16 && tdtype != NTK_DT_F32) return NTK_E_DTYPE;
+    if (T < 0 || vocab <= 0 || width <= 0 || pos0 < 0) return NTK_E_SHAPE;
+    if (T == 0) return NTK_OK;
+    const dim3 grid(((width + 1) / 2 + 255) / 256, T);
+    if (tdtype == NTK_DT_BF16)
+        hipLaunchKernelGGL(embed_sinusoid_kernel<uint16_t>, grid, dim3(256), 0, resolve_stream(stream), out, (const uint16_t*)table, tokens, vocab, width, scale, freq, pos0);
+    else
+        hipLaunchKernelGGL(embed_sinusoid_kernel<float>, grid, dim3(256), 0, resolve_stream(stream), out, (const float*)table, tokens, vocab, width, scale, freq, pos0);
     return last_launch_status();
 }
 

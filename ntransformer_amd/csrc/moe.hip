@@ -14,7 +14,7 @@ constexpr int kMaxExperts = 256;
 // one workgroup per token: its 16 waves share the experts (wave w: experts w, w + 16, ...), a lane requests its whole part of the router row before
 // it uses any of it; thread 0 then does the softmax and the `top` picks over the scores in LDS
 constexpr int kRouteThreads = 1024;
-struct RouteForm { int score, groups, keep, group_top, renorm; float scale; };
+struct RouteForm { int score, groups, keep, group_top, renorm; float scale; const float* correction; const float* add_y; int ld_add; const float* add_w; float add_eps; };
 
 // the largest of a wave's 4 x 64 values (lane l holds entries l, l + 64, l + 128, l + 192); equal values: the lower index
 __device__ __forceinline__ void wave_argmax4(const float (&v)[4], int lane, float& bv, int& bi) {
@@ -31,14 +31,27 @@ __device__ __forceinline__ void wave_argmax4(const float (&v)[4], int lane, floa
     }
 }
 
-__global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, float* wts, float* sgate, const float* h, int ldh, const float* wr, const float* wsg,
+__global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, float* wts, float* sgate, float* h, int ldh, const float* wr, const float* wsg,
                                                                  int n, int E, int top, const RouteForm f) {
     __shared__ float z[kMaxExperts];
     extern __shared__ __attribute__((aligned(16))) float xs[];   // the token's row
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = kRouteThreads / 64;
     const long long t = blockIdx.x;
-    const float* x = h + t * ldh;
-    for (int k = threadIdx.x; k < n; k += kRouteThreads) xs[k] = x[k];
+    float* x = h + t * ldh;
+    if (f.add_y) {     // (uniform) what the row is still owed joins it: y / rms(y) * w; a thread re-reads its own entries
+        __shared__ float red[16];
+        const float* y = f.add_y + t * f.ld_add;
+        float ss = 0.0f;
+        for (int k = threadIdx.x; k < n; k += kRouteThreads) { xs[k] = x[k]; ss = fmaf(y[k], y[k], ss); }
+        const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)n + f.add_eps);
+        for (int k = threadIdx.x; k < n; k += kRouteThreads) {
+            const float v = fmaf(y[k] * inv, f.add_w[k], xs[k]);
+            xs[k] = v;
+            x[k] = v;
+        }
+    } else {
+        for (int k = threadIdx.x; k < n; k += kRouteThreads) xs[k] = x[k];
+    }
     __syncthreads();
     const bool vec = (n % 4 == 0) && !((uintptr_t)wr & 15) && !(wsg && ((uintptr_t)wsg & 15));
     for (int e = wave; e < E + (wsg ? 1 : 0); e += nw) {
@@ -71,16 +84,22 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, floa
         m = wave_max(m);
         den = 0.0f;
 #pragma unroll
-        for (int c = 0; c < 4; ++c) { v[c] = lane + 64 * c < E ? expf(v[c] - m) : -1.0f; den += fmaxf(v[c], 0.0f); }
+        for (int c = 0; c < 4; ++c) { v[c] = lane + 64 * c < E ? expf(v[c] - m) : -INFINITY; den += fmaxf(v[c], 0.0f); }
         den = wave_sum(den);
     } else {
 #pragma unroll
-        for (int c = 0; c < 4; ++c) v[c] = lane + 64 * c < E ? 1.0f / (1.0f + expf(-z[lane + 64 * c])) : -1.0f;
+        for (int c = 0; c < 4; ++c) v[c] = lane + 64 * c < E ? 1.0f / (1.0f + expf(-z[lane + 64 * c])) : -INFINITY;
+    }
+    if (f.correction) {     // (uniform) what is chosen by is no longer what is weighted with: the scores stay in LDS, v becomes the choice scores
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+            if (lane + 64 * c < E) { const float s = v[c] / den; z[lane + 64 * c] = s; v[c] = s + f.correction[lane + 64 * c]; }
+        __builtin_amdgcn_wave_barrier();
     }
     __shared__ int pick_id[kMaxExperts];
     __shared__ float pick_sc[kMaxExperts];
     if (f.groups > 1) {
-        // group scores: lane l owns groups l, l + 64, ...: the sum of the group's `group_top` largest scores (scores are >= 0; taken ones are marked -1)
+        // group scores: lane l owns groups l, l + 64, ...: the sum of the group's `group_top` largest scores (taken ones are marked -inf)
         __shared__ float sc[kMaxExperts];
         __shared__ unsigned char open_group[kMaxExperts];
 #pragma unroll
@@ -92,13 +111,13 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, floa
 #pragma unroll
         for (int c = 0; c < 4; ++c) {
             const int g = lane + 64 * c;
-            gs[c] = -1.0f;
+            gs[c] = -INFINITY;
             if (g < f.groups) {
                 float sum = 0.0f;
                 int taken[8];
                 const int nt = min(min(f.group_top, per), 8);
                 for (int k = 0; k < nt; ++k) {
-                    float best = -1.0f;
+                    float best = -INFINITY;
                     int bi = -1;
                     for (int e = g * per; e < (g + 1) * per; ++e) {
                         bool used = false;
@@ -118,22 +137,22 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, floa
             int bi;
             wave_argmax4(gs, lane, bv, bi);
             if (lane == 0) open_group[bi] = 1;
-            if ((bi & 63) == lane) gs[bi >> 6] = -2.0f;
+            if ((bi & 63) == lane) gs[bi >> 6] = -INFINITY;
         }
         __builtin_amdgcn_wave_barrier();
 #pragma unroll
         for (int c = 0; c < 4; ++c)
-            if (lane + 64 * c < E && !open_group[(lane + 64 * c) / per]) v[c] = -1.0f;
+            if (lane + 64 * c < E && !open_group[(lane + 64 * c) / per]) v[c] = -INFINITY;
     }
     float chosen = 0.0f;
     for (int s = 0; s < top; ++s) {
         float bv;
         int bi;
         wave_argmax4(v, lane, bv, bi);
-        const float sc1 = bv / den;
+        const float sc1 = f.correction ? z[bi] : bv / den;
         chosen += sc1;
         if (lane == 0) { pick_id[s] = bi; pick_sc[s] = sc1; }
-        if ((bi & 63) == lane) v[bi >> 6] = -2.0f;
+        if ((bi & 63) == lane) v[bi >> 6] = -INFINITY;
     }
     const float mul = (f.renorm ? 1.0f / (chosen + 1e-20f) : 1.0f) * f.scale;
     for (int s = lane; s < top; s += 64) { ids[t * top + s] = pick_id[s]; wts[t * top + s] = pick_sc[s] * mul; }   // (same wave wrote them: in order)
@@ -201,12 +220,16 @@ __global__ void clipped_glu_kernel(float* a, int lda, const float* gu, int ldgu,
 
 template <bool ADD>
 __global__ void moe_combine_kernel(float* x, const float* mix, const float* d, const int* where, const float* wts, const float* shared, const float* sgate,
-                                   int top, int n) {
+                                   int top, int n, const int* ids, int n_experts, const float* h, int ldh) {
     const long long t = blockIdx.y;
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n) return;
     float s = 0.0f;
-    for (int k = 0; k < top; ++k) s = fmaf(wts[t * top + k], d[(long long)where[t * top + k] * n + i], s);
+    for (int k = 0; k < top; ++k) {
+        const long long p = t * top + k;
+        const float* row = ids && ids[p] >= n_experts ? h + t * ldh : d + (long long)(where ? where[p] : p) * n;   // an identity expert gives the input back
+        s = fmaf(wts[p], row[i], s);
+    }
     if (shared) s = sgate ? fmaf(sgate[t], shared[t * n + i], s) : s + shared[t * n + i];
     if (mix) s += mix[t * n + i];
     if constexpr (ADD) x[t * n + i] += s; else x[t * n + i] = s;
@@ -218,7 +241,9 @@ using namespace ntk;
 
 int ntk_moe_route(int* ids, float* wts, float* sgate, const float* h, int ldh, const float* w_router, const float* shared_gate_w, int T, int n, int E, int top,
                   void* stream) {
-    const ntk_route_desc r{0, 1, 1, 1, 1, 1.0f};   // softmax scores, no groups, weights renormalised over the chosen
+    ntk_route_desc r{};
+    r.groups = r.keep = r.group_top = r.renorm = 1;
+    r.scale = 1.0f;   // softmax scores, no groups, weights renormalised over the chosen
     return ntk_moe_route_ex(ids, wts, sgate, h, ldh, w_router, shared_gate_w, T, n, E, top, &r, stream);
 }
 
@@ -227,12 +252,13 @@ int ntk_moe_route_ex(int* ids, float* wts, float* sgate, const float* h, int ldh
     if (!ids || !wts || !h || !w_router || !r) return NTK_E_NULL;
     if (T < 0 || n <= 0 || E <= 0 || E > kMaxExperts || top <= 0 || top > E || ldh < n) return NTK_E_SHAPE;
     if (r->score != 0 && r->score != 1) return NTK_E_SHAPE;
+    if (r->add_y && (!r->add_w || r->ld_add < n || r->add_y == h)) return NTK_E_SHAPE;
     const int groups = r->groups > 1 ? r->groups : 1;
     if (groups > 1 && (E % groups || r->keep < 1 || r->keep > groups || r->group_top < 1 || r->group_top > 8 || (long long)r->keep * (E / groups) < top)) return NTK_E_SHAPE;
     if (T == 0) return NTK_OK;
     if ((size_t)n * 4 > 128 * 1024) return NTK_E_SHAPE;
-    const RouteForm f{r->score, groups, r->keep, r->group_top, r->renorm, r->scale};
-    hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(kRouteThreads), (size_t)n * 4, resolve_stream(stream), ids, wts, sgate, h, ldh, w_router, shared_gate_w, n, E, top, f);
+    const RouteForm f{r->score, groups, r->keep, r->group_top, r->renorm, r->scale, r->correction, r->add_y, r->ld_add, r->add_w, r->add_eps};
+    hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(kRouteThreads), (size_t)n * 4, resolve_stream(stream), ids, wts, sgate, (float*)h, ldh, w_router, shared_gate_w, n, E, top, f);
     return last_launch_status();
 }
 
@@ -270,14 +296,22 @@ int ntk_moe_combine(float* x, const float* mix, const float* d, const int* where
     if (!x || !d || !where || !wts || (shared && !sgate)) return NTK_E_NULL;
     if (T < 0 || top <= 0 || n <= 0) return NTK_E_SHAPE;
     if (T == 0) return NTK_OK;
-    hipLaunchKernelGGL(moe_combine_kernel<true>, dim3((n + 255) / 256, T), dim3(256), 0, resolve_stream(stream), x, mix, d, where, wts, shared, sgate, top, n);
+    hipLaunchKernelGGL(moe_combine_kernel<true>, dim3((n + 255) / 256, T), dim3(256), 0, resolve_stream(stream), x, mix, d, where, wts, shared, sgate, top, n,
+                       (const int*)nullptr, 0, (const float*)nullptr, 0);
     return last_launch_status();
 }
 
 int ntk_moe_sum(float* out, const float* d, const int* where, const float* wts, const float* shared, const float* sgate, int T, int top, int n, void* stream) {
-    if (!out || !d || !where || !wts) return NTK_E_NULL;
-    if (T < 0 || top <= 0 || n <= 0) return NTK_E_SHAPE;
+    if (!where) return NTK_E_NULL;
+    return ntk_moe_sum_ex(out, d, where, nullptr, 0, nullptr, 0, wts, shared, sgate, T, top, n, stream);
+}
+
+int ntk_moe_sum_ex(float* out, const float* d, const int* where, const int* ids, int n_experts, const float* h, int ldh, const float* wts, const float* shared,
+                   const float* sgate, int T, int top, int n, void* stream) {
+    if (!out || !d || !wts || (ids && !h)) return NTK_E_NULL;
+    if (T < 0 || top <= 0 || n <= 0 || (ids && ldh < n)) return NTK_E_SHAPE;
     if (T == 0) return NTK_OK;
-    hipLaunchKernelGGL(moe_combine_kernel<false>, dim3((n + 255) / 256, T), dim3(256), 0, resolve_stream(stream), out, (const float*)nullptr, d, where, wts, shared, sgate, top, n);
+    hipLaunchKernelGGL(moe_combine_kernel<false>, dim3((n + 255) / 256, T), dim3(256), 0, resolve_stream(stream), out, (const float*)nullptr, d, where, wts, shared, sgate, top, n,
+                       ids, n_experts, h, ldh);
     return last_launch_status();
 }

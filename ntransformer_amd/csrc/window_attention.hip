@@ -1,6 +1,7 @@
 // window_attention.hip -- grouped-query softmax attention over a cache of rotated keys and values: causal, optional sliding window, one or two score
 // maps per head over the same values (two maps: the differential pair out = a_0 - lambda * a_1), optional unit norm of every head's output, optional
-// learned bias by bucketed distance on the scaled score (a table of distances -> buckets, a table of buckets x heads), optional cap on the score
+// learned bias by bucketed distance on the scaled score (a table of distances -> buckets, a table of buckets x heads) or a bias that falls with the distance at
+// a rate of the head's, optional cap on the score
 // (cap * tanh(score / cap)), optional sink (a key without a value in every softmax: of score 0, or of a learned score per head), optional gate on the output
 // (element by element or one number per head); beside the sliding window the first `keep_first` positions can stay visible for ever, and instead of it there is a
 // mask of chunks (a query sees the keys of its own chunk of `window` positions, counted from position 0, up to itself).
@@ -95,6 +96,58 @@ __global__ __launch_bounds__(NT) void window_prepare_kernel(const PrepareArgs a)
     }
 }
 
+// One wave per (token, vector): RMS norm of every head's vector on its own with one shared weight, query temperature behind the norm, rotation; the values are copied
+// (they may be the keys as they were projected).  A lane re-reads and rewrites its own entries or pairs only, after the wave's sum has used all of them.
+__global__ __launch_bounds__(256) void window_prepare_heads_kernel(const PrepareArgs a, int G) {
+    const int lane = threadIdx.x & 63, j = blockIdx.y * 4 + (threadIdx.x >> 6), dn = a.dn, dv = a.nv / G;
+    const int t = blockIdx.x, pos = a.pos0 + t, nk = a.k ? a.nk : 0;
+    if (j >= a.nq + nk + (a.k ? G : 0)) return;
+    if (j >= a.nq + nk) {                                     // a value vector
+        const int o = (j - a.nq - nk) * dv;
+        const float* vt = a.v + (long long)t * a.ldv + o;
+        float* dst = a.cache + (long long)pos * a.row + nk * dn + o;
+        for (int i = lane; i < dv; i += 64) dst[i] = vt[i] + (a.vb ? a.vb[o + i] : 0.0f);
+        return;
+    }
+    const bool is_q = j < a.nq;
+    const int o = (is_q ? j : j - a.nq) * dn;
+    const float* src = is_q ? a.q + (long long)t * a.ldq + o : a.k + (long long)t * a.ldk + o;
+    float* dst = is_q ? a.q + (long long)t * a.ldq + o : a.cache + (long long)pos * a.row + o;
+    const float* b = is_q ? a.qb : a.kb;
+    const float* w = is_q ? a.q_norm : a.k_norm;
+    constexpr int KEEP = 4;                                   // a lane's first entries stay in registers
+    float v[KEEP];
+    float ss = 0.0f;
+#pragma unroll
+    for (int u = 0; u < KEEP; ++u) {
+        const int i = lane + 64 * u;
+        v[u] = i < dn ? src[i] + (b ? b[o + i] : 0.0f) : 0.0f;
+        ss = fmaf(v[u], v[u], ss);
+    }
+    for (int i = lane + 64 * KEEP; i < dn; i += 64) { const float x = src[i] + (b ? b[o + i] : 0.0f); ss = fmaf(x, x, ss); }
+    const float inv = w ? 1.0f / sqrtf(wave_sum(ss) / (float)dn + a.norm_eps) : 1.0f;
+    const float temp = is_q && a.temp_coef != 0.0f ? 1.0f + a.temp_coef * logf((float)floor((double)(pos + 1) / a.temp_every) + 1.0f) : 1.0f;
+    auto formed = [&](float x, int i) { x = w ? x * inv * w[i] : x; return is_q ? x * temp : x; };
+    if (a.dims == 0) {
+#pragma unroll
+        for (int u = 0; u < KEEP; ++u)
+            if (lane + 64 * u < dn) dst[lane + 64 * u] = formed(v[u], lane + 64 * u);
+        for (int i = lane + 64 * KEEP; i < dn; i += 64) dst[i] = formed(src[i] + (b ? b[o + i] : 0.0f), i);
+        return;
+    }
+    const int half = a.dims / 2, pair = a.halves ? half : 1, step = a.halves ? 1 : 2;   // pair i = entries (i * step, i * step + pair)
+    for (int i = lane; i < half; i += 64) {
+        const int e = step * i;
+        const double ang = (double)pos * a.freq[i];
+        float ra, rb;
+        rope_rotate(formed(src[e] + (b ? b[o + e] : 0.0f), e), formed(src[e + pair] + (b ? b[o + e + pair] : 0.0f), e + pair), (float)(cos(ang) * (double)a.mag),
+                    (float)(sin(ang) * (double)a.mag), ra, rb);
+        dst[e] = ra;
+        dst[e + pair] = rb;
+    }
+    for (int i = a.dims + lane; i < dn; i += 64) dst[i] = formed(src[i] + (b ? b[o + i] : 0.0f), i);
+}
+
 struct WinArgs {
     float* out; int ldo;
     const float* q; int ldq;
@@ -108,6 +161,7 @@ struct WinArgs {
     const float* gate; int ldg, head_gate;                // gate != NULL: out[t][h][c] *= sigmoid(gate[t * ldg + h * dv + c]), or gate[t * ldg + h] with head_gate
     int keep;                                             // positions 0 .. keep - 1 stay visible behind the sliding window
     const float* sinks;                                   // the sink's score per head (NULL with `sink`: 0)
+    const float* slopes;                                  // slopes[head] * distance comes off the scaled score
 };
 
 // first key a query at position p sees
@@ -175,11 +229,13 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
     }
     float mx[M][WQPW], l[M][WQPW], acc[M][WQPW][WMAXC];
     int rpos[WQPW], rhead[WQPW];
+    float slope[WQPW];
 #pragma unroll
     for (int i = 0; i < WQPW; ++i) {
         const int rho = row0 + wave * WQPW + i;
         rpos[i] = rho < n_rows ? a.pos0 + rho / R : -1;
         rhead[i] = g * R + rho % R;
+        slope[i] = a.slopes ? a.slopes[rhead[i]] : 0.0f;
         // the sink is a key without a value: the running maximum and sum start from it (in the first part only when the keys are split)
         const bool sunk = (a.sink || a.sinks) && (a.splits <= 1 || blockIdx.z == 0);
         const float sink_score = a.sinks ? a.sinks[rhead[i]] : 0.0f;
@@ -234,6 +290,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(const WinArgs a) 
                 const bool vis = lane < nk && rpos[i] >= 0 && j <= rpos[i] && (j >= first_visible(rpos[i], a.window, a.chunks) || j < a.keep);
                 float sv = vis ? s[i] * a.scale : -INFINITY;
                 if (a.rel && vis) sv += a.rel[(long long)a.bucket_of[min(rpos[i] - j, a.n_dist - 1)] * a.H + rhead[i]];
+                if (a.slopes && vis) sv -= slope[i] * (float)(rpos[i] - j);
                 if (a.softcap > 0.0f && vis) sv = a.softcap * tanhf(sv / a.softcap);
                 const float mn = fmaxf(mx[m][i], wave_max(sv));
                 const float ms = mn == -INFINITY ? 0.0f : mn;
@@ -398,6 +455,12 @@ int ntk_window_prepare_ex(const ntk_window_prepare_desc* d, void* stream) {
                         rot->layout == NTK_ROT_HALVES ? 1 : 0, d->pos0, d->qb, d->kb, d->vb, d->temp_coef, d->temp_every, d->v_other, d->ld_other, d->v_blend, d->v_keep,
                         d->ld_keep, d->q_norm, d->k_norm, d->norm_eps};
     const size_t lds = (size_t)(rot->dims + 2) * sizeof(float);
+    if (d->head_norm) {
+        if (d->v_other || d->v_keep) return NTK_E_SHAPE;      // (that form does not blend values)
+        const int vectors = d->H * d->maps + (d->k ? d->G * d->maps + d->G : 0);
+        hipLaunchKernelGGL(window_prepare_heads_kernel, dim3(d->T, (vectors + 3) / 4), dim3(256), 0, resolve_stream(stream), a, d->G);
+        return last_launch_status();
+    }
     // a normed row is read twice, the second time behind a sum over the workgroup: few tokens (decoding) take workgroups of 1024
     if ((d->q_norm || d->k_norm) && d->T <= 32) hipLaunchKernelGGL(window_prepare_kernel<1024>, dim3(d->T), dim3(1024), lds, resolve_stream(stream), a);
     else hipLaunchKernelGGL(window_prepare_kernel<256>, dim3(d->T), dim3(256), lds, resolve_stream(stream), a);
@@ -425,7 +488,7 @@ int ntk_window_attention(const ntk_window_attention_desc* d, void* stream) {
     if (d->gate && d->ldg < (d->head_gate ? d->H : d->H * d->dv)) return NTK_E_SHAPE;
     a.gate = d->gate; a.ldg = d->ldg; a.head_gate = d->head_gate ? 1 : 0;
     if (d->keep_first < 0 || (d->keep_first > 0 && a.chunks)) return NTK_E_SHAPE;
-    a.keep = d->keep_first; a.sinks = d->sinks;
+    a.keep = d->keep_first; a.sinks = d->sinks; a.slopes = d->slopes;
     a.splits = d->scratch ? window_splits(d->T, d->H, d->G, window_keys(d->pos0, d->T, d->window, a.chunks, a.keep)) : 1;
     a.scratch = d->scratch;
     a.rel = d->rel; a.bucket_of = d->bucket_of; a.n_dist = d->n_dist;

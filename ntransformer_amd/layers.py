@@ -19,7 +19,9 @@ class DenseDesc(C.Structure):
     _fields_ = [("Y", C.c_void_p), ("ldy", C.c_int), ("X", C.c_void_p), ("ldx", C.c_int), ("W", C.c_void_p), ("wstride", C.c_longlong), ("wdtype", C.c_int),
                 ("offsets", C.c_void_p), ("G", C.c_int), ("rows", C.c_void_p), ("row_div", C.c_int), ("T", C.c_int), ("N", C.c_int), ("K", C.c_int),
                 ("accumulate", C.c_int), ("glu_ff", C.c_int), ("glu_limit", C.c_float), ("glu_alpha", C.c_float),
-                ("norm_w", C.c_void_p), ("norm_eps", C.c_float), ("norm_offset", C.c_float), ("glu_up_offset", C.c_float), ("glu_cubic", C.c_float)]
+                ("norm_w", C.c_void_p), ("norm_eps", C.c_float), ("norm_offset", C.c_float), ("glu_up_offset", C.c_float), ("glu_cubic", C.c_float),
+                ("act", C.c_int), ("add_y", C.c_void_p), ("ld_add", C.c_int), ("add_w", C.c_void_p), ("add_eps", C.c_float), ("add_mult", C.c_float),
+                ("x_out", C.c_void_p), ("ldxo", C.c_int)]
 
 
 class Rotary(C.Structure):
@@ -35,7 +37,7 @@ class WindowPrepareDesc(C.Structure):
                 ("H", C.c_int), ("G", C.c_int), ("maps", C.c_int), ("dn", C.c_int), ("dv", C.c_int), ("rot", C.POINTER(Rotary)),
                 ("qb", C.c_void_p), ("kb", C.c_void_p), ("vb", C.c_void_p), ("temp_coef", C.c_float), ("temp_every", C.c_double),
                 ("v_other", C.c_void_p), ("ld_other", C.c_int), ("v_blend", C.c_float), ("v_keep", C.c_void_p), ("ld_keep", C.c_int), ("pos0", C.c_int), ("T", C.c_int),
-                ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("norm_eps", C.c_float)]
+                ("q_norm", C.c_void_p), ("k_norm", C.c_void_p), ("norm_eps", C.c_float), ("head_norm", C.c_int)]
 
 
 class WindowAttentionDesc(C.Structure):
@@ -43,7 +45,7 @@ class WindowAttentionDesc(C.Structure):
                 ("H", C.c_int), ("G", C.c_int), ("maps", C.c_int), ("dn", C.c_int), ("dv", C.c_int), ("pos0", C.c_int), ("T", C.c_int), ("window", C.c_int),
                 ("scale", C.c_float), ("lam", C.c_float), ("sub_norm", C.c_int), ("eps", C.c_float), ("out_scale", C.c_float), ("scratch", C.c_void_p),
                 ("rel", C.c_void_p), ("bucket_of", C.c_void_p), ("n_dist", C.c_int), ("mask_mode", C.c_int), ("softcap", C.c_float), ("sink", C.c_int),
-                ("gate", C.c_void_p), ("ldg", C.c_int), ("head_gate", C.c_int), ("keep_first", C.c_int), ("sinks", C.c_void_p)]
+                ("gate", C.c_void_p), ("ldg", C.c_int), ("head_gate", C.c_int), ("keep_first", C.c_int), ("sinks", C.c_void_p), ("slopes", C.c_void_p)]
 
 
 class GatedSeamDesc(C.Structure):
@@ -65,7 +67,17 @@ DECAY_GIVEN, DECAY_SIGMOID_ROOT, DECAY_EXP_SIGMOID, DECAY_EXP_SOFTPLUS = 0, 1, 2
 
 
 class RouteDesc(C.Structure):
-    _fields_ = [("score", C.c_int), ("groups", C.c_int), ("keep", C.c_int), ("group_top", C.c_int), ("renorm", C.c_int), ("scale", C.c_float)]
+    _fields_ = [("score", C.c_int), ("groups", C.c_int), ("keep", C.c_int), ("group_top", C.c_int), ("renorm", C.c_int), ("scale", C.c_float), ("correction", C.c_void_p),
+                ("add_y", C.c_void_p), ("ld_add", C.c_int), ("add_w", C.c_void_p), ("add_eps", C.c_float)]
+
+
+class MoeFewDesc(C.Structure):
+    _fields_ = [("out", C.c_void_p), ("ldo", C.c_int), ("h", C.c_void_p), ("ldh", C.c_int), ("ids", C.c_void_p), ("wts", C.c_void_p), ("top", C.c_int), ("experts", C.c_int),
+                ("up", C.c_void_p), ("down", C.c_void_p), ("ff", C.c_int), ("shared_up", C.c_void_p), ("shared_down", C.c_void_p), ("shared_ff", C.c_int), ("sgate", C.c_void_p),
+                ("wdtype", C.c_int), ("act", C.c_int), ("mid", C.c_void_p), ("T", C.c_int), ("n", C.c_int)]
+
+
+ACT_NONE, ACT_RELU2 = 0, 1
 
 
 def _bind():
@@ -74,6 +86,10 @@ def _bind():
         return L
     vp, i, f, ll = C.c_void_p, C.c_int, C.c_float, C.c_longlong
     L.ntk_dense.argtypes = [C.POINTER(DenseDesc), vp]
+    L.ntk_embed_sinusoid.argtypes = [vp, vp, i, vp, i, i, i, f, vp, i, vp]
+    L.ntk_latent_fold_query_prepare.argtypes = [vp, vp, i, vp, i, i, i, i, i, vp, i, vp, i, vp, f, i, vp]
+    L.ntk_moe_few.argtypes = [C.POINTER(MoeFewDesc), vp]
+    L.ntk_moe_sum_ex.argtypes = [vp, vp, vp, vp, i, vp, i, vp, vp, vp, i, i, i, vp]
     L.ntk_dense_linear.argtypes = [vp, i, vp, i, vp, i, i, i, i, i, vp]
     L.ntk_embed_dense.argtypes = [vp, vp, i, vp, i, i, i, vp]
     L.ntk_rmsnorm_offset.argtypes = [vp, vp, vp, vp, i, vp, i, i, i, f, f, vp]
@@ -163,9 +179,10 @@ def _i(a) -> DeviceBuffer:
 
 def dense(x: np.ndarray, w: np.ndarray, dtype: str = "float32", offsets=None, rows=None, row_div: int = 1, n_rows: Optional[int] = None,
           y0: Optional[np.ndarray] = None, glu_limit: Optional[float] = None, glu_alpha: float = 1.702, norm_w: Optional[np.ndarray] = None,
-          norm_eps: float = 1e-6, norm_offset: float = 0.0, glu_up_offset: float = 1.0, glu_cubic: float = 0.0) -> np.ndarray:
+          norm_eps: float = 1e-6, norm_offset: float = 0.0, glu_up_offset: float = 1.0, glu_cubic: float = 0.0, act: int = ACT_NONE, add=None):
     """y[r] = x[src(r)] . w[g(r)]^T; w [N, K] or a stack [G, N, K] with `offsets` [G + 1]; rows: source row per output row (divided by row_div);
-    y0: start values to accumulate onto."""
+    y0: start values to accumulate onto; act: an activation on the result; add (few rows) = (add_y, add_w, eps, mult): the rows are first x + mult * rms(add_y) * add_w
+    -> (y, those rows)."""
     L = _bind()
     w = np.asarray(w)
     stacked = w.ndim == 3
@@ -180,12 +197,18 @@ def dense(x: np.ndarray, w: np.ndarray, dtype: str = "float32", offsets=None, ro
     nb = _f(norm_w) if norm_w is not None else None
     if nb is not None:          # fused RMS norm of the activation rows (few rows)
         d.norm_w, d.norm_eps, d.norm_offset = nb.ptr, norm_eps, norm_offset
+    d.act = act
+    if add is not None:
+        ab, awb, xo = _f(add[0]), _f(add[1]), DeviceBuffer.zeros(T * K * 4)
+        d.add_y, d.ld_add, d.add_w, d.add_eps, d.add_mult, d.x_out, d.ldxo = ab.ptr, K, awb.ptr, add[2], add[3], xo.ptr, K
     if glu_limit is not None:   # fused clipped GLU (few rows): N / 2 outputs per row
         d.glu_ff, d.glu_limit, d.glu_alpha, d.ldy = N // 2, glu_limit, glu_alpha, N // 2
         check(L.ntk_dense(C.byref(d), None), "ntk_dense")
-        return yb.numpy(np.float32, T * (N // 2)).reshape(T, N // 2)
-    check(L.ntk_dense(C.byref(d), None), "ntk_dense")
-    return yb.numpy(np.float32, T * N).reshape(T, N)
+        N //= 2
+    else:
+        check(L.ntk_dense(C.byref(d), None), "ntk_dense")
+    y = yb.numpy(np.float32, T * N).reshape(T, N)
+    return (y, xo.numpy(np.float32, T * K).reshape(T, K)) if add is not None else y
 
 
 def rmsnorm_offset(x: np.ndarray, w1: np.ndarray, w2: Optional[np.ndarray], eps: float, offset: float):
@@ -392,10 +415,10 @@ def window_prepare_biased(q, k, v, H: int, G: int, dn: int, dv: int, pos0: int, 
 def window_attention(q: np.ndarray, cache: np.ndarray, H: int, G: int, maps: int, dn: int, dv: int, pos0: int, window: int, scale: float, lam: float = 0.0,
                      sub_norm: bool = False, eps: float = 1e-6, out_scale: float = 1.0, split: bool = True, rel: Optional[np.ndarray] = None,
                      bucket_of: Optional[np.ndarray] = None, chunks: bool = False, softcap: float = 0.0, sink: bool = False, gate: Optional[np.ndarray] = None,
-                     keep_first: int = 0, sinks: Optional[np.ndarray] = None, head_gate: bool = False) -> np.ndarray:
+                     keep_first: int = 0, sinks: Optional[np.ndarray] = None, head_gate: bool = False, slopes: Optional[np.ndarray] = None) -> np.ndarray:
     """q [T, H * maps * dn] (rotated), cache rows [G][maps][dn] keys | [G][dv] values; split: long key ranges of few rows may be cut into merged parts;
     rel [buckets, H] with bucket_of [distances]: a bias by distance on the scaled score; keep_first: positions that stay visible beside the window;
-    sinks [H]: the sink's score per head; gate [T, H * dv], or [T, H] with head_gate"""
+    sinks [H]: the sink's score per head; gate [T, H * dv], or [T, H] with head_gate; slopes [H]: slopes[h] * distance comes off the scaled score"""
     L = _bind()
     T, row = q.shape[0], G * (maps * dn + dv)
     qb, cb = _f(q), _f(cache)
@@ -411,6 +434,9 @@ def window_attention(q: np.ndarray, cache: np.ndarray, H: int, G: int, maps: int
     if sinks is not None:
         kb = _f(sinks)
         d.sinks = kb.ptr
+    if slopes is not None:
+        slb = _f(slopes)
+        d.slopes = slb.ptr
     if gate is not None:        # a sigmoid gate on the result
         gb = _f(gate)
         d.gate, d.ldg, d.head_gate = gb.ptr, gate.shape[1], int(head_gate)
@@ -437,15 +463,23 @@ def lightning_attention(q: np.ndarray, k: np.ndarray, v: np.ndarray, decay, H: i
 
 
 def moe_route_ex(h: np.ndarray, w_router: np.ndarray, top: int, score: int = 1, groups: int = 1, keep: int = 1, group_top: int = 2, renorm: bool = False,
-                 scale: float = 1.0):
+                 scale: float = 1.0, correction: Optional[np.ndarray] = None, add=None):
+    """correction [E]: joins the scores when groups and experts are chosen; add = (add_y, add_w, eps): the rows are first h + rms(add_y) * add_w -> (ids, weights, those rows)"""
     L = _bind()
     T, n = h.shape
     E = w_router.shape[0]
     hb, wb = _f(h), _f(w_router)
     ids, wts = DeviceBuffer.zeros(T * top * 4), DeviceBuffer.zeros(T * top * 4)
     r = RouteDesc(score, groups, keep, group_top, int(renorm), scale)
+    if correction is not None:
+        cb = _f(correction)
+        r.correction = cb.ptr
+    if add is not None:
+        ab, awb = _f(add[0]), _f(add[1])
+        r.add_y, r.ld_add, r.add_w, r.add_eps = ab.ptr, n, awb.ptr, add[2]
     check(L.ntk_moe_route_ex(ids.ptr, wts.ptr, None, hb.ptr, n, wb.ptr, None, T, n, E, top, C.byref(r), None), "ntk_moe_route_ex")
-    return ids.numpy(np.int32, T * top).reshape(T, top), wts.numpy(np.float32, T * top).reshape(T, top)
+    out = ids.numpy(np.int32, T * top).reshape(T, top), wts.numpy(np.float32, T * top).reshape(T, top)
+    return out + (hb.numpy(np.float32, T * n).reshape(T, n),) if add is not None else out
 
 
 def glu(gu: np.ndarray, limit: float = float("inf"), alpha: float = 1.0, up_offset: float = 0.0) -> np.ndarray:
@@ -457,14 +491,20 @@ def glu(gu: np.ndarray, limit: float = float("inf"), alpha: float = 1.0, up_offs
     return out.numpy(np.float32, rows * ff).reshape(rows, ff)
 
 
-def moe_sum(d, where, wts, shared=None, sgate=None) -> np.ndarray:
+def moe_sum(d, where, wts, shared=None, sgate=None, ids=None, n_experts: int = 0, h=None) -> np.ndarray:
+    """ids [T, top] with h [T, n]: pairs of experts >= n_experts give the input h back; where None: pair p is row p of d"""
     L = _bind()
     T, top = wts.shape
     n = d.shape[1]
-    db, wb, tb = _f(d), _i(where), _f(wts)
+    db, wb, tb = _f(d), (_i(where) if where is not None else None), _f(wts)
     sb = _f(shared) if shared is not None else None
     gb = _f(sgate) if sgate is not None else None
     out = DeviceBuffer.zeros(T * n * 4)
+    if ids is not None or where is None:
+        ib, hb = (_i(ids) if ids is not None else None), (_f(h) if h is not None else None)
+        check(L.ntk_moe_sum_ex(out.ptr, db.ptr, wb.ptr if wb else None, ib.ptr if ib else None, n_experts, hb.ptr if hb else None, n, tb.ptr, sb.ptr if sb else None,
+                               gb.ptr if gb else None, T, top, n, None), "ntk_moe_sum_ex")
+        return out.numpy(np.float32, T * n).reshape(T, n)
     check(L.ntk_moe_sum(out.ptr, db.ptr, wb.ptr, tb.ptr, sb.ptr if sb else None, gb.ptr if gb else None, T, top, n, None), "ntk_moe_sum")
     return out.numpy(np.float32, T * n).reshape(T, n)
 
@@ -576,9 +616,10 @@ def glu_cubic(gu: np.ndarray, ff: int, alpha: float, cubic: float, limit: float 
 
 def window_prepare_ex(q, k, v, H: int, G: int, dn: int, dv: int, pos0: int, freq=None, dims: int = 0, layout: int = ROT_NEIGHBOURS, v_other=None, v_blend: float = 0.0,
                       keep: bool = False, cache: Optional[np.ndarray] = None, cache_rows: Optional[int] = None, mag: float = 1.0, q_norm=None, k_norm=None,
-                      norm_eps: float = 1e-6, qb=None, kb=None):
+                      norm_eps: float = 1e-6, qb=None, kb=None, head_norm: bool = False, temp_coef: float = 0.0, temp_every: float = 1.0, values_are_keys: bool = False):
     """one score map: (biases,) norms over the whole q / k with the weights q_norm / k_norm, rotation by `layout`, values blended with v_other [T, G * dv] on their
-    way into the cache rows -> (cache, q, the values as they came if keep); k None: queries only (the cache comes back as it was)"""
+    way into the cache rows -> (cache, q, the values as they came if keep); k None: queries only (the cache comes back as it was); head_norm: q_norm / k_norm [dn], every
+    head normed on its own, ahead of the query temperature; values_are_keys: v is k's memory"""
     L = _bind()
     T, row = q.shape[0], G * (dn + dv)
     n = cache_rows or (pos0 + T)
@@ -592,8 +633,9 @@ def window_prepare_ex(q, k, v, H: int, G: int, dn: int, dv: int, pos0: int, freq
     d = WindowPrepareDesc()
     d.cache, d.row, d.q, d.ldq = cb.ptr, row, qd.ptr, q.shape[1]
     if k is not None:
-        d.k, d.ldk, d.v, d.ldv = kd.ptr, k.shape[1], vd.ptr, v.shape[1]
-    d.H, d.G, d.maps, d.dn, d.dv, d.rot, d.temp_every, d.pos0, d.T = H, G, 1, dn, dv, C.pointer(rot), 1.0, pos0, T
+        d.k, d.ldk, d.v, d.ldv = (kd.ptr, k.shape[1], kd.ptr, k.shape[1]) if values_are_keys else (kd.ptr, k.shape[1], vd.ptr, v.shape[1])
+    d.H, d.G, d.maps, d.dn, d.dv, d.rot, d.temp_every, d.pos0, d.T = H, G, 1, dn, dv, C.pointer(rot), temp_every, pos0, T
+    d.temp_coef, d.head_norm = temp_coef, int(head_norm)
     d.q_norm, d.k_norm, d.norm_eps, d.qb, d.kb = ptr(qn), ptr(kn), norm_eps, ptr(qbias), ptr(kbias)
     if ob:
         d.v_other, d.ld_other, d.v_blend = ob.ptr, G * dv, v_blend
@@ -613,6 +655,45 @@ def embed_bigram(table: np.ndarray, bigram: np.ndarray, tokens, prev: int, pos0:
     out = DeviceBuffer.zeros(T * W * 4)
     check(L.ntk_embed_bigram(out.ptr, tb.ptr, bb.ptr, dt, ib.ptr, prev, pos0, T, V, W, scale, bigram.shape[0] - 1, mul_prev, mul_cur, None), "ntk_embed_bigram")
     return out.numpy(np.float32, T * W).reshape(T, W)
+
+
+def embed_sinusoid(table: np.ndarray, tokens, pos0: int, freq: np.ndarray, scale: float = 1.0, dtype: str = "float32") -> np.ndarray:
+    """table [vocab, width] -> [T, width]: the tokens' rows plus the sinusoidal position vectors of positions pos0 .. with the frequencies freq [(width + 1) / 2]"""
+    L = _bind()
+    T, (V, W) = len(tokens), table.shape
+    (tb, dt), ib, fb = weight_buffer(table, dtype), _i(tokens), DeviceBuffer.from_numpy(np.ascontiguousarray(freq, np.float64))
+    out = DeviceBuffer.zeros(T * W * 4)
+    check(L.ntk_embed_sinusoid(out.ptr, tb.ptr, dt, ib.ptr, T, V, W, scale, fb.ptr, pos0, None), "ntk_embed_sinusoid")
+    return out.numpy(np.float32, T * W).reshape(T, W)
+
+
+def latent_fold_query_prepare(q: np.ndarray, w_uk: np.ndarray, heads: int, dn: int, kv: np.ndarray, norm_w: np.ndarray, eps: float, pos0: int, cache: np.ndarray,
+                              dtype: str = "float32"):
+    """q [T, H * dn], kv [T, R] raw latents -> (folded queries [T, H * R], cache [rows, R] with rows pos0 .. normed in)"""
+    L = _bind()
+    T, R = q.shape[0], w_uk.shape[1]
+    qb, (wb, dt), kb, nb, cb = _f(q), weight_buffer(w_uk, dtype), _f(kv), _f(norm_w), _f(cache)
+    out = DeviceBuffer.zeros(T * heads * R * 4)
+    check(L.ntk_latent_fold_query_prepare(out.ptr, qb.ptr, q.shape[1], wb.ptr, dt, T, heads, dn, R, cb.ptr, cache.shape[1], kb.ptr, kv.shape[1], nb.ptr, eps, pos0, None),
+          "ntk_latent_fold_query_prepare")
+    return out.numpy(np.float32, T * heads * R).reshape(T, heads * R), cb.numpy(np.float32, cache.size).reshape(cache.shape)
+
+
+def moe_few(h: np.ndarray, ids, wts, up: np.ndarray, down: np.ndarray, shared_up=None, shared_down=None, sgate=None, act: int = ACT_RELU2, dtype: str = "float32") -> np.ndarray:
+    """h [T, n], ids / wts [T, top], up [E, ff, n], down [E, n, ff], shared_up [sff, n], shared_down [n, sff], sgate [T] -> the weighted sum of the chosen units [T, n]"""
+    L = _bind()
+    T, n = h.shape
+    E, ff = up.shape[:2]
+    top, sff = ids.shape[1], (shared_up.shape[0] if shared_up is not None else 0)
+    hb, ib, tb = _f(h), _i(ids), _f(wts)
+    (ub, dt), (db, _) = weight_buffer(up, dtype), weight_buffer(down, dtype)
+    su, sd = (weight_buffer(w, dtype)[0] if w is not None else None for w in (shared_up, shared_down))
+    gb = _f(sgate) if sgate is not None else None
+    out, mid = DeviceBuffer.zeros(T * n * 4), DeviceBuffer.from_numpy(np.full(T * (top * ff + sff), np.nan, np.float32))
+    d = MoeFewDesc(out.ptr, n, hb.ptr, n, ib.ptr, tb.ptr, top, E, ub.ptr, db.ptr, ff, su.ptr if su else None, sd.ptr if sd else None, sff, gb.ptr if gb else None, dt, act,
+                   mid.ptr, T, n)
+    check(L.ntk_moe_few(C.byref(d), None), "ntk_moe_few")
+    return out.numpy(np.float32, T * n).reshape(T, n)
 
 
 def glu_rows(gu: np.ndarray, ff: int, lda: int, limit: float = float("inf"), alpha: float = 1.0, cubic: float = 0.0, up_offset: float = 0.0) -> np.ndarray:

@@ -179,10 +179,11 @@ def tubazen_shapes(cfg: dict, buckets: int = 32, rank: int = 64) -> Dict[str, Tu
     return s
 
 
-def fifotar_config(preset: str, layers: int = 4, mlp_everywhere: bool = True, attention_only: bool = False) -> dict:
+def fifotar_config(preset: str, layers: int = 4, mlp_everywhere: bool = True, attention_only: bool = False,
+                   order: Tuple[str, ...] = ("attention", "delta", "latent_attention", "delta")) -> dict:
     """the scaled family at the preset's width, heads and vocabulary: chunked attention (four query heads per key/value head, chunks of the preset's window,
     capped scores, blended values), the per-head delta rule (two value heads per key head, keys and values of the preset's sizes, four taps) and latent
-    attention (the preset's ranks) in the order attention, delta, latent, delta (attention_only: nothing but the first); the clipped gated feed-forward with the
+    attention (the preset's ranks) in the order given, over and over (attention_only: nothing but attention); the clipped gated feed-forward with the
     bytes of the gated family's"""
     p = PRESETS[preset]
     H, dn, dv = p["heads"], p["dim"], p["vdim"]
@@ -190,16 +191,14 @@ def fifotar_config(preset: str, layers: int = 4, mlp_everywhere: bool = True, at
     ff -= ff % 64
     ls = []
     for k in range(layers):
-        if k % 4 == 0 or attention_only:
+        t = "attention" if attention_only else order[k % len(order)]
+        if t == "attention":
             mx = {"heads": H, "kv_heads": max(H // 4, 1), "dim": dn, "vdim": dv, "scale": 1.0 / math.sqrt(dn), "softcap": 40.0, "mask": {"size": p["window"]}, "v_mix": True}
-            t = "attention"
-        elif k % 4 == 2:
+        elif t == "latent_attention":
             mx = {"heads": H, "dim": dn, "rot_dim": p["rot_dim"], "vdim": dv, "kv_rank": p["kv_rank"], "q_rank": p["q_rank"], "scale": 1.0 / math.sqrt(dn + p["rot_dim"]),
                   "rot": {"base": 1000000.0, "dims": p["rot_dim"], "scaling": {"factor": 8.0, "original": 4096, "fast": 16.0, "slow": 2.0}}}
-            t = "latent_attention"
         else:
             mx = {"heads": H, "kv_heads": max(H // 2, 1), "dim": dn, "vdim": dv, "conv": 4}
-            t = "delta"
         has_mlp = mlp_everywhere or t != "delta"
         ls.append({"type": t, "mixer": mx, "mlp": {"kind": "dense", "ff": max(ff, 64), "limit": 7.0} if has_mlp else None})
     return {"architecture": "Fifotar", "layers": ls, "norm": {"eps": 1e-5}, "embedding": {"scale": math.sqrt(p["width"])}, "residual_mult": 0.7, "logit_softcap": 25.0,
@@ -273,10 +272,69 @@ def zalazen_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
     return s
 
 
+def gibevik_config(preset: str, layers: int = 4) -> dict:
+    """the post-norm family at the preset's width, heads and vocabulary: a latent layer (the preset's latent size), one that reads its latents, then two layers of
+    grouped-query attention (four query heads per key/value head), over and over; every first of a pair with the dense gated feed-forward of fifotar_config, every second
+    with the preset's mixture as plain units (the same bytes per token), a sixteenth of the router's choices being the identity, four groups of which two are kept"""
+    p = PRESETS[preset]
+    H, dn, dv = p["heads"], p["dim"], p["vdim"]
+    ff = (p["top"] * p["ff"] + p["shared_ff"]) * 2 // 3
+    ff -= ff % 64
+    grouped = p["experts"] % 4 == 0 and p["experts"] // 2 >= p["top"]
+    identity = max(p["experts"] // 16, 1)
+    ls = []
+    for k in range(layers):
+        if k % 4 < 2:
+            t, mx = "latent_attention", {"heads": H, "dim": dn, "vdim": dv, "kv_rank": p["kv_rank"], "scale": 1.0 / math.sqrt(dn)}
+            if k % 4 == 1:
+                mx["kv_from"] = k - 1
+        else:
+            t, mx = "attention", {"heads": H, "kv_heads": max(H // 4, 1), "dim": dn, "vdim": dn, "scale": 1.0 / math.sqrt(dn), "q_temp": {"coef": 0.1, "every": 512}}
+        if k % 2 == 0:
+            ml = {"kind": "dense", "ff": max(ff, 64)}
+        else:
+            ml = {"kind": "moe", "expert": {"ff": p["ff"]}, "router": {"experts": p["experts"] - identity, "identity": identity, "top": p["top"]}, "shared": {"ff": p["shared_ff"]}}
+            if grouped:
+                ml["router"]["groups"] = {"count": 4, "keep": 2}
+        ls.append({"type": t, "mixer": mx, "mlp": ml})
+    return {"architecture": "Gibevik", "layers": ls, "norm": {"eps": 1e-5}, "vocab": p["vocab"], "width": p["width"]}
+
+
+def gibevik_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
+    W, V = cfg["width"], cfg["vocab"]
+    s: Dict[str, Tuple[int, ...]] = {"embed": (V, W), "head": (V, W), "final.norm": (W,)}
+    for i, L in enumerate(cfg["layers"]):
+        p, mx, ml = "l%d." % i, L["mixer"], L.get("mlp")
+        H, dn, dv, q = mx["heads"], mx["dim"], mx["vdim"], p + "mix."
+        s[p + "norm1"], s[q + "q"], s[q + "o"] = (W,), (H * dn, W), (W, H * dv)
+        if L["type"] == "attention":
+            s[q + "k"], s[q + "q.norm"], s[q + "k.norm"], s[q + "g"] = (mx.get("kv_heads", H) * dn, W), (dn,), (dn,), (H * dv, W)
+        else:
+            R = mx["kv_rank"]
+            if mx.get("kv_from") is None:
+                s[q + "dkv"], s[q + "dkv.norm"] = (R, W), (R,)
+            s[q + "uk"], s[q + "uv"], s[q + "g"] = (H * dn, R), (H * dv, R), (H, W)
+        if not ml:
+            continue
+        s[p + "norm2"] = (W,)
+        if ml["kind"] == "dense":
+            s[p + "mlp.gate"], s[p + "mlp.up"], s[p + "mlp.down"] = (ml["ff"], W), (ml["ff"], W), (W, ml["ff"])
+            continue
+        rt, ff = ml["router"], ml["expert"]["ff"]
+        for e in range(rt["experts"]):
+            s["%smlp.e%d.up" % (p, e)], s["%smlp.e%d.down" % (p, e)] = (ff, W), (W, ff)
+        n = rt["experts"] + rt.get("identity", 0)
+        s[p + "mlp.router"], s[p + "mlp.correction"] = (n, W), (n,)
+        if ml.get("shared"):
+            sf = ml["shared"]["ff"]
+            s[p + "mlp.shared.up"], s[p + "mlp.shared.down"], s[p + "mlp.shared.sg"] = (sf, W), (W, sf), (1, W)
+    return s
+
+
 def shapes_of(cfg: dict) -> Dict[str, Tuple[int, ...]]:
     arch = cfg.get("architecture")
     return (nizorax_shapes(cfg) if arch == "Nizorax" else tubazen_shapes(cfg) if arch == "Tubazen" else fifotar_shapes(cfg) if arch == "Fifotar" else
-            zalazen_shapes(cfg) if arch == "Zalazen" else
+            zalazen_shapes(cfg) if arch == "Zalazen" else gibevik_shapes(cfg) if arch == "Gibevik" else
             fabolorn_shapes(cfg))
 
 
@@ -317,7 +375,7 @@ def write_folder(folder: str, cfg: dict, seed: int = 20260925) -> int:
                     around_one = name.rsplit(".", 1)[-1] in ("norm", "norm1", "norm2")
                 if cfg.get("architecture") == "Nizorax":     # layer-norm weights around one, biases / lambda vectors / activation numbers small
                     around_one = name.rsplit(".", 1)[-1] in ("norm", "norm1", "norm2", "norm1b", "norm2b")
-                if cfg.get("architecture") in ("Fifotar", "Zalazen"):     # every norm weight is stored plain; decay rates and biases small
+                if cfg.get("architecture") in ("Fifotar", "Zalazen", "Gibevik"):     # every norm weight is stored plain; decay rates and biases small
                     around_one = "norm" in name.rsplit(".", 1)[-1]
                 vals = 0.1 * pool[:n] + (1.0 if around_one else 0.0)
                 f.write(_bf16(vals).tobytes())
