@@ -131,7 +131,7 @@ struct GemvParams {
 template <int DT, bool A16> struct Dot;
 
 typedef float f32x2 __attribute__((ext_vector_type(2)));
-// two FMAs per instruction (v_pk_fma_f32): the dot products are VALU-issue bound for the 4/5/6-bit formats
+// two independent sums: the dot products are VALU-issue bound for the 4/5/6-bit formats
 __device__ __forceinline__ f32x2 pkfma(f32x2 a, f32x2 b, f32x2 c) { return __builtin_elementwise_fma(a, b, c); }
 // hide a value from the optimiser so that (x & 0x0F0F0F0F) stays ONE v_and and each byte converts with
 // v_cvt_f32_ubyteN (otherwise hipcc re-derives every nibble with its own v_bfe_u32 + v_cvt_f32_ubyte0)
