@@ -352,6 +352,8 @@ typedef struct ntk_route_desc {
 } ntk_route_desc;
 int ntk_moe_route_ex(int* ids, float* wts, float* sgate, const float* h, int ldh, const float* w_router, const float* shared_gate_w, int T, int n, int E, int top,
                      const ntk_route_desc* r, void* stream);
+/* The choice alone, from router outputs that a product left: z [T][ldz] = [E outputs | the shared unit's gate ahead of its sigmoid (if sgate)] (r->add_y must be NULL) */
+int ntk_moe_pick(int* ids, float* wts, float* sgate, const float* z, int ldz, int T, int E, int top, const ntk_route_desc* r, void* stream);
 /* The experts of a few tokens (T <= ntk_dense_few_rows(), decoding) in two launches, without grouping: plain units U_e then D_e with the activation `act` between them,
  *   out[t] = sum_s wts[t][s] * D_e act(U_e h[t])  (e = ids[t][s]; e >= experts: wts[t][s] * h[t])  + sgate[t] * Ds act(Us h[t])   (shared_up may be NULL; sgate NULL: 1)
  * up [experts][ff][n], down [experts][n][ff], shared_up [shared_ff][n], shared_down [n][shared_ff], all of dtype wdtype; mid: work space F32 [T][top * ff + shared_ff].

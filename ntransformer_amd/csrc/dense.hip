@@ -1,13 +1,15 @@
 // dense.hip -- products with dense weight matrices (bfloat16 or float32, row-major [out][in]) for the layer-list model families.
 //
-// One entry point (ntk_dense) and three kernel forms behind it:
+// One entry point for a product (ntk_dense) with three kernel forms behind it:
 //   * dense_mfma_kernel   bf16 weights, more than kGemvRows rows: 128 x 128 / 64 x 128 / 64 x 64 output tiles on v_mfma_f32_16x16x32_bf16; the F32 activations are rounded
 //                         to bfloat16 (nearest even) on their way into LDS, sums stay F32 in the accumulators;
 //   * dense_fma_kernel    float32 weights, more than kGemvRows rows: the same tiling with plain F32 FMAs, k ascending (true 32-bit);
 //   * dense_gemv_kernel   up to kGemvRows rows (decoding): every wave streams a few weight rows at once, 16 bytes per lane and row, the activation
-//                         row sits in LDS; bf16 weights are widened exactly and multiplied in F32.
+//                         row sits in LDS; bf16 weights are widened exactly and multiplied in F32.  What runs inside the launch on the way in: what the row is still owed (a
+//                         sublayer's normed output), an RMS norm; on the way out: a gated unit or an activation.
 // Rows can be grouped (a mixture of experts: sorted rows of group g take matrix g) and gathered (row r reads activation row rows[r] / row_div).
 // Group sizes live on the device, so the grid covers the worst case and workgroups outside their group's range leave at once.
+// A second entry point (ntk_moe_few) runs all of a few tokens' chosen experts, the shared unit and their weighted sum in two row-streaming launches.
 #include "common.hip.h"
 #include "../../include/ntk_layers.h"
 
@@ -464,7 +466,7 @@ template <typename WT> __device__ __forceinline__ float weight_value(const WT* p
     if constexpr (sizeof(WT) == 2) return bf2f(*p); else return *p;
 }
 
-// mid[t][slot * ff + f] = act(U_e h)[f] for the token's chosen experts, then the shared unit's; grid (rows / (4 RW), T)
+// mid[t][slot * ff + f] = act(U_e h)[f] times the expert's weight for the token's chosen experts, then the shared unit's times its gate; grid (rows / (4 RW), T)
 template <typename WT, int RW>
 __global__ __launch_bounds__(256) void moe_few_up_kernel(const MoeFewArgs a) {
     extern __shared__ __attribute__((aligned(16))) float xs[];   // the token's row
@@ -516,44 +518,57 @@ __global__ __launch_bounds__(256) void moe_few_up_kernel(const MoeFewArgs a) {
 #pragma unroll
     for (int i = 0; i < RW; ++i) {
         s[i] = wave_sum_lane63(s[i]);
-        if (lane == 63 && w[i]) a.mid[(long long)t * rows + m0 + i] = activate(s[i], a.act);
+        if (lane == 63 && w[i]) {
+            const float wt = m0 + i < routed ? a.wts[(long long)t * a.top + (m0 + i) / a.ff] : a.sgate ? a.sgate[t] : 1.0f;
+            a.mid[(long long)t * rows + m0 + i] = activate(s[i], a.act) * wt;
+        }
     }
 }
 
-// out[t][i] = one row of weights [D_e0[i] | D_e1[i] | ... | Ds[i]] against the activations side by side, each times its expert's weight; grid (n / (4 RW), T)
-template <typename WT, int RW>
+// out[t][i] = one row of weights [D_e0[i] | D_e1[i] | ... | Ds[i]] against the weighted activations side by side; grid (n / (4 RW), T).  A wave goes through the
+// row in passes of 512 entries inside one segment (a chosen expert, the shared unit; identity experts are passed over), with the requests of DEPTH passes under way.
+template <typename WT, int RW, int DEPTH>
 __global__ __launch_bounds__(256) void moe_few_down_kernel(const MoeFewArgs a) {
-    extern __shared__ __attribute__((aligned(16))) float xs[];   // [top * ff + shared_ff] weighted activations
+    extern __shared__ __attribute__((aligned(16))) float xs[];   // [top * ff + shared_ff]
     const int t = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int routed = a.top * a.ff, K = routed + a.shared_ff, i0 = (blockIdx.x * 4 + wave) * RW;
     const int* ids = a.ids + (long long)t * a.top;
-    const float* wts = a.wts + (long long)t * a.top;
-    int row[RW];
+    const float* mid = a.mid + (long long)t * K;
+    long long row[RW];
 #pragma unroll
     for (int i = 0; i < RW; ++i) row[i] = min(i0 + i, a.n - 1);     // (rows past the end re-read the last one and are not stored)
-    // where a lane stands in the concatenated row: segment (slot; `top` = the shared unit) and place in it
-    int slot = 0, off = 0;
-    auto settle = [&]() { while (slot < a.top && off >= a.ff) { off -= a.ff; ++slot; } };
-    WeightPiece<WT> cur[RW], next[RW];
-    auto request = [&](WeightPiece<WT>(&p)[RW]) {
-        const WT* base = nullptr;
-        long long step = 0;
-        if (slot < a.top) {
-            const int e = ids[slot];
-            if (e >= 0 && e < a.experts) { base = (const WT*)a.down + (long long)e * a.n * a.ff + off; step = a.ff; }
-        } else if (off < a.shared_ff) {
-            base = (const WT*)a.shared_down + off; step = a.shared_ff;
+    // the pass that is requested next: segment (`top` = the shared unit, top + 1 = past the end), its matrix, the pass's first entry in it -- uniform over the wave
+    int seg = -1, k0 = 0, len = 0;
+    const WT* mat = nullptr;
+    auto next_segment = [&]() {
+        for (++seg, k0 = 0; seg < a.top; ++seg) {
+            const int e = ids[seg];
+            if (e >= 0 && e < a.experts) { mat = (const WT*)a.down + (long long)e * a.n * a.ff; len = a.ff; return; }
         }
-#pragma unroll
-        for (int i = 0; i < RW; ++i) { if (base) p[i].load(base + row[i] * step); else p[i].clear(); }
+        if (seg == a.top && a.shared_ff > 0) { mat = (const WT*)a.shared_down; len = a.shared_ff; return; }
+        seg = a.top + 1;
     };
-    if (a.vec) { off = lane * 8; settle(); request(cur); }
-    for (int m = tid; m < K; m += 256) {
-        const int sl = m / a.ff;                              // (beyond the routed part: >= top)
-        float wt = a.sgate ? a.sgate[t] : 1.0f;
-        bool live = true;
-        if (m < routed) { const int e = ids[sl]; wt = wts[sl]; live = e >= 0 && e < a.experts; }
-        xs[m] = live ? a.mid[(long long)t * K + m] * wt : 0.0f;     // (an identity expert's part of the work space is not written)
+    WeightPiece<WT> piece[DEPTH][RW];
+    int at[DEPTH];                                            // the lane's first activation of the pass (-1: none; -2: no pass)
+    auto request = [&](WeightPiece<WT>(&p)[RW], int& x_at) {
+        x_at = -2;
+        if (seg > a.top) return;
+        const int k = k0 + lane * 8;
+        x_at = k < len ? (seg < a.top ? seg * a.ff : routed) + k : -1;
+        if (x_at >= 0)
+#pragma unroll
+            for (int i = 0; i < RW; ++i) p[i].load(mat + row[i] * len + k);
+        k0 += 512;
+        if (k0 >= len) next_segment();
+    };
+    next_segment();
+    if (a.vec)
+#pragma unroll
+        for (int d = 0; d < DEPTH; ++d) request(piece[d], at[d]);
+    if (a.vec) {
+        for (int m = 4 * tid; m < K; m += 4 * 256) *reinterpret_cast<float4*>(xs + m) = *reinterpret_cast<const float4*>(mid + m);
+    } else {
+        for (int m = tid; m < K; m += 256) xs[m] = mid[m];
     }
     __syncthreads();
     if (i0 >= a.n) return;                                    // (uniform over the wave)
@@ -561,29 +576,27 @@ __global__ __launch_bounds__(256) void moe_few_down_kernel(const MoeFewArgs a) {
 #pragma unroll
     for (int i = 0; i < RW; ++i) s[i] = 0.0f;
     if (a.vec) {
-        for (int k = lane * 8; k < K; k += 512) {
-            if (k + 512 < K) { off += 512; settle(); request(next); }
+        bool more = true;
+        while (more) {
 #pragma unroll
-            for (int i = 0; i < RW; ++i) { s[i] = cur[i].dot(xs + k, s[i]); cur[i] = next[i]; }
+            for (int d = 0; d < DEPTH; ++d) {
+                if (at[d] >= 0) {
+#pragma unroll
+                    for (int i = 0; i < RW; ++i) s[i] = piece[d][i].dot(xs + at[d], s[i]);
+                }
+                more = at[d] != -2;
+                if (more) request(piece[d], at[d]);
+            }
         }
     } else {
-        for (int k = lane; k < K; k += 64) {
-            const WT* base;
-            long long step;
-            if (k < routed) {
-                const int e = ids[k / a.ff];
-                if (e < 0 || e >= a.experts) continue;
-                base = (const WT*)a.down + (long long)e * a.n * a.ff + k % a.ff; step = a.ff;
-            } else {
-                base = (const WT*)a.shared_down + (k - routed); step = a.shared_ff;
-            }
+        for (; seg <= a.top; next_segment())
+            for (int k = lane; k < len; k += 64)
 #pragma unroll
-            for (int i = 0; i < RW; ++i) s[i] = fmaf(weight_value(base + row[i] * step), xs[k], s[i]);
-        }
+                for (int i = 0; i < RW; ++i) s[i] = fmaf(weight_value(mat + row[i] * len + k), xs[(seg < a.top ? seg * a.ff : routed) + k], s[i]);
     }
     float ident = 0.0f;                                       // the weights of the token's identity experts
     for (int sl = 0; sl < a.top; ++sl)
-        if (ids[sl] >= a.experts) ident += wts[sl];
+        if (ids[sl] >= a.experts) ident += a.wts[(long long)t * a.top + sl];
 #pragma unroll
     for (int i = 0; i < RW; ++i) {
         s[i] = wave_sum_lane63(s[i]);
@@ -591,13 +604,14 @@ __global__ __launch_bounds__(256) void moe_few_down_kernel(const MoeFewArgs a) {
     }
 }
 
+constexpr int kMoeDepth = 8;
 template <typename WT>
 static void launch_moe_few(const MoeFewArgs& a, int T, hipStream_t s) {
     const int rows = a.top * a.ff + a.shared_ff;
-    constexpr int RW = 2;
-    const dim3 gu((rows + 4 * RW - 1) / (4 * RW), T), gd((a.n + 4 * RW - 1) / (4 * RW), T);
-    hipLaunchKernelGGL((moe_few_up_kernel<WT, RW>), gu, dim3(256), ((size_t)a.n * 4 + 15) & ~(size_t)15, s, a);
-    hipLaunchKernelGGL((moe_few_down_kernel<WT, RW>), gd, dim3(256), ((size_t)rows * 4 + 15) & ~(size_t)15, s, a);
+    const size_t lu = ((size_t)a.n * 4 + 15) & ~(size_t)15, ld = ((size_t)rows * 4 + 15) & ~(size_t)15;
+    hipLaunchKernelGGL((moe_few_up_kernel<WT, 2>), dim3((rows + 7) / 8, T), dim3(256), lu, s, a);
+    if ((long long)a.n * T >= 4096) hipLaunchKernelGGL((moe_few_down_kernel<WT, 2, kMoeDepth>), dim3((a.n + 7) / 8, T), dim3(256), ld, s, a);
+    else hipLaunchKernelGGL((moe_few_down_kernel<WT, 1, kMoeDepth>), dim3((a.n + 3) / 4, T), dim3(256), ld, s, a);
 }
 
 template <typename WT, bool ADD>
@@ -697,7 +711,9 @@ int ntk_moe_few(const ntk_moe_few_desc* d, void* stream) {
             !(((uintptr_t)d->h | (uintptr_t)d->up | (uintptr_t)d->down | (uintptr_t)d->shared_up | (uintptr_t)d->shared_down) & 15);
     static bool raised = false;     // (idempotent: a race sets the same attributes twice)
     if (!raised) {
-        const void* fn[] = {(const void*)moe_few_up_kernel<uint16_t, 2>, (const void*)moe_few_up_kernel<float, 2>, (const void*)moe_few_down_kernel<uint16_t, 2>, (const void*)moe_few_down_kernel<float, 2>};
+        const void* fn[] = {(const void*)moe_few_up_kernel<uint16_t, 2>, (const void*)moe_few_up_kernel<float, 2>, 
+                            (const void*)moe_few_down_kernel<uint16_t, 2, kMoeDepth>, (const void*)moe_few_down_kernel<float, 2, kMoeDepth>,
+                            (const void*)moe_few_down_kernel<uint16_t, 1, kMoeDepth>, (const void*)moe_few_down_kernel<float, 1, kMoeDepth>};
         for (const void* f : fn) NTK_HIP_TRY(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, NTK_MOE_FEW_MID * 4));
         raised = true;
     }

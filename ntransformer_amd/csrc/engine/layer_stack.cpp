@@ -825,6 +825,11 @@ int LayerStackModel::upload_mlp(const ModelFolder& f, const std::string& p, int 
         if (M.shared.gate_up.out_f != M.shared.in_rows() || M.shared.down.out_f != W) return fail(NTK_E_SHAPE, li + ": shared expert matrices do not have the configured sizes");
         if (form_.shared_gate) LS_TRY(upload_vector(f, p + "mlp.shared.sg", W, &M.shared_gate));
     }
+    if (form_.post_norm && f.tensor(p + "mlp.router")->dtype == "BF16" && (!M.has_shared || f.tensor(p + "mlp.shared.sg")->dtype == "BF16")) {     // (stored values: no rounding)
+        const uint64_t counted = weight_bytes_;      // (a second copy of tensors that are counted already)
+        LS_TRY(upload_matrix(f, M.has_shared ? std::vector<std::string>{p + "mlp.router", p + "mlp.shared.sg"} : std::vector<std::string>{p + "mlp.router"}, W, M.choose));
+        weight_bytes_ = counted;
+    }
     return NTK_OK;
 }
 
@@ -994,7 +999,7 @@ int LayerStackModel::alloc_buffers() {
     if (form_.scaled)
         ok = ok && fl(&ff_, C * W) && fl(&zf_, C * std::max(max_ffn_, 1)) && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc) && fl(&rscratch_, rsc) &&
              fl(&cv_, C * std::max(max_conv_, 1)) && fl(&vfirst_, C * std::max(max_gv_, 1));
-    if (form_.post_norm) ok = ok && fl(&ff_, C * W) && fl(&zf_, C * std::max(max_ffn_, 1)) && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc) && fl(&mid_, (size_t)ntk_dense_few_rows() * max_mid_);
+    if (form_.post_norm) ok = ok && fl(&ff_, C * W) && fl(&zf_, C * std::max(max_ffn_, 1)) && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc) && fl(&mid_, (size_t)ntk_dense_few_rows() * max_mid_) && fl(&rz_, (size_t)ntk_dense_few_rows() * (max_e_ + 1));
     if (form_.dense_parallel) ok = ok && fl(&gu2_, C * 2 * std::max(max_ffn_, 1)) && fl(&wscratch_, wsc);
     want_dev_ = tokens_dev_ ? tokens_dev_ + C : nullptr;   // one staging area: [tokens of a pass | wanted places], filled by ONE stream-ordered copy from pinned memory
     h_stage_ = (int*)nt_hip_malloc_host(2 * C * sizeof(int));
@@ -1189,20 +1194,28 @@ int LayerStackModel::run_moe(const StackLayer& L, const float* h, int T, bool in
     const MoeFeedForward& M = L.mlp;
     const int W = info_.width, choices = M.experts + M.identity;
     float* sgate = M.has_shared && M.shared_gate ? sg_ : nullptr;
-    ntk_route_desc route = M.route;
-    if (form_.post_norm && owed_.y) {      // what the stream is still owed joins it in the router's launch
-        route.add_y = owed_.y; route.ld_add = W; route.add_w = owed_.nb.w; route.add_eps = eps_;
-        owed_.y = nullptr;
-    }
-    LS_TRY(ntk_moe_route_ex(ids_, wts_, sgate, h, W, M.router, sgate ? M.shared_gate : nullptr, T, W, choices, M.top, &route, stream_));
     const size_t mid = (size_t)M.top * M.routed.ff + (M.has_shared ? M.shared.ff : 0);
-    if (M.routed.plain && T <= ntk_dense_few_rows() && mid <= NTK_MOE_FEW_MID && W <= NTK_MOE_FEW_MID && !into_stream) {     // decoding: two launches for all of a token's units
+    if (M.choose.ptr && T <= ntk_dense_few_rows() && mid <= NTK_MOE_FEW_MID && W <= NTK_MOE_FEW_MID && !into_stream) {
+        // decoding: the router and the shared unit's gate as one product (with what the stream is still owed inside it), the choice, two launches for all of a token's units
+        const int nz = (int)M.choose.out_f;
+        ntk_dense_desc z{};
+        z.Y = rz_; z.ldy = nz; z.X = h; z.ldx = W; z.W = M.choose.ptr; z.wdtype = M.choose.dtype; z.G = 1; z.row_div = 1; z.T = T; z.N = nz; z.K = W;
+        const bool stream_in = h == x_;
+        LS_TRY(first_product(z));
+        if (stream_in) h = x_;             // (the product may have left the stream in its other buffer)
+        LS_TRY(ntk_moe_pick(ids_, wts_, sgate, rz_, nz, T, choices, M.top, &M.route, stream_));
         ntk_moe_few_desc d{};
         d.out = ff_; d.ldo = W; d.h = h; d.ldh = W; d.ids = ids_; d.wts = wts_; d.top = M.top; d.experts = M.experts; d.up = M.routed.gate_up.ptr; d.down = M.routed.down.ptr; d.ff = M.routed.ff;
         if (M.has_shared) { d.shared_up = M.shared.gate_up.ptr; d.shared_down = M.shared.down.ptr; d.shared_ff = M.shared.ff; d.sgate = sgate; }
         d.wdtype = M.routed.down.dtype; d.act = NTK_ACT_RELU2; d.mid = mid_; d.T = T; d.n = W;
         return ntk_moe_few(&d, stream_);
     }
+    ntk_route_desc route = M.route;
+    if (form_.post_norm && owed_.y) {      // what the stream is still owed joins it in the router's launch
+        route.add_y = owed_.y; route.ld_add = W; route.add_w = owed_.nb.w; route.add_eps = eps_;
+        owed_.y = nullptr;
+    }
+    LS_TRY(ntk_moe_route_ex(ids_, wts_, sgate, h, W, M.router, sgate ? M.shared_gate : nullptr, T, W, choices, M.top, &route, stream_));
     LS_TRY(ntk_moe_group(offsets_, order_, where_, ids_, T, M.top, choices, stream_));     // (identity experts come last: rows behind offsets_[experts], which no product visits)
     LS_TRY(run_experts(M.glu_alpha, M.glu_up_offset, M.routed, h, gu_, act_, dn_, T * M.top, offsets_, order_, M.top));
     if (M.has_shared) LS_TRY(run_experts(M.glu_alpha, M.glu_up_offset, M.shared, h, sgu_, sact_, sdn_, T, nullptr, nullptr, 1));

@@ -201,6 +201,7 @@ struct MoeFeedForward {
     bool has_shared = false;
     GatedExperts shared;
     float* shared_gate = nullptr;     // F32 [width]; none: the shared expert is added as it is
+    DenseW choose;                    // post-norm form: [router rows ; shared gate row] as one matrix for few tokens (the router's values, exact in either dtype)
 };
 
 struct DenseFeedForward {             // down(act(up h)), act = a N(z) + b N(z^2) + c N(z^3) + e
@@ -375,7 +376,7 @@ private:
     float *x_ = nullptr, *x0_ = nullptr, *cat_ = nullptr, *h1_ = nullptr, *h2_ = nullptr, *a_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *qf_ = nullptr, *lat_ = nullptr,
           *att_ = nullptr, *kx_ = nullptr, *vx_ = nullptr, *mix_ = nullptr, *wts_ = nullptr, *sg_ = nullptr, *gu_ = nullptr, *act_ = nullptr, *dn_ = nullptr,
           *sgu_ = nullptr, *sact_ = nullptr, *sdn_ = nullptr, *scratch_ = nullptr, *xw_ = nullptr, *hn_ = nullptr, *hist_ = nullptr, *ff_ = nullptr, *zf_ = nullptr, *wscratch_ = nullptr, *lscratch_ = nullptr,
-          *results_ = nullptr, *zq_ = nullptr, *gu2_ = nullptr, *rscratch_ = nullptr, *cv_ = nullptr, *vfirst_ = nullptr, *mid_ = nullptr;   // gated form: the layer results of the pass [runs + 1][chunk][width], decay pre-activations, [gate | up | residual gate]
+          *results_ = nullptr, *zq_ = nullptr, *gu2_ = nullptr, *rscratch_ = nullptr, *cv_ = nullptr, *vfirst_ = nullptr, *mid_ = nullptr, *rz_ = nullptr;   // gated form: the layer results of the pass [runs + 1][chunk][width], decay pre-activations, [gate | up | residual gate]
     size_t max_mid_ = 0;              // (post-norm form: the experts' activations of a token side by side)
     int max_rec_ = 0, max_gu2_ = 0, max_conv_ = 0, max_gv_ = 0;   // (scaled form: convolution channels, key heads x value size of the blending attention layers)
     int *ids_ = nullptr, *offsets_ = nullptr, *order_ = nullptr, *where_ = nullptr, *tokens_dev_ = nullptr, *want_dev_ = nullptr;

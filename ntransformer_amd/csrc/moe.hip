@@ -1,5 +1,6 @@
-// moe.hip -- the routing side of a mixture of experts: router scores and the choice (F32), the stable grouping of (token, slot) pairs by expert that
-// the grouped product (dense.hip) consumes, the clipped gated activation between an expert's two products, and the weighted sum back into the
+// moe.hip -- the routing side of a mixture of experts: router scores and the choice (F32; optionally by score plus a learned correction, optionally among the best groups
+// only; in one launch, or the choice alone behind a product), the stable grouping of (token, slot) pairs by expert that
+// the grouped product (dense.hip) consumes, the clipped gated activation between an expert's two products, and the weighted sum (identity experts: of the input itself) back into the
 // residual stream.  The experts' products themselves are ntk_dense calls over the stacked expert matrices.
 //
 // A token's result never depends on the other tokens of the launch: the grouping only decides WHERE a pair's row sits, each row is computed on its
@@ -18,17 +19,97 @@ struct RouteForm { int score, groups, keep, group_top, renorm; float scale; cons
 
 // the largest of a wave's 4 x 64 values (lane l holds entries l, l + 64, l + 128, l + 192); equal values: the lower index
 __device__ __forceinline__ void wave_argmax4(const float (&v)[4], int lane, float& bv, int& bi) {
-    bv = v[0];
-    bi = lane;
+    bv = wave_max(fmaxf(fmaxf(v[0], v[1]), fmaxf(v[2], v[3])));
+    bi = 0;
 #pragma unroll
-    for (int c = 1; c < 4; ++c)
-        if (v[c] > bv) { bv = v[c]; bi = lane + 64 * c; }      // (equal values: the lower index stays)
-#pragma unroll
-    for (int o = 32; o >= 1; o >>= 1) {
-        const float ov = __shfl_xor(bv, o, 64);
-        const int oi = __shfl_xor(bi, o, 64);
-        if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+    for (int c = 3; c >= 0; --c) {                            // (the lowest index is the first lane of the first quarter that holds the value)
+        const unsigned long long m = __ballot(v[c] == bv);
+        if (m) bi = 64 * c + __ffsll((unsigned long long)m) - 1;
     }
+}
+
+// scores and the picks by one wave: lane l holds experts l, l + 64, l + 128, l + 192; z [E] in LDS
+__device__ __forceinline__ void pick_experts(float* z, int lane, long long t, int E, int top, const RouteForm& f, int* ids, float* wts) {
+    float v[4];
+    float den = 1.0f;
+    if (f.score == 0) {
+        float m = -INFINITY;
+#pragma unroll
+        for (int c = 0; c < 4; ++c) { v[c] = lane + 64 * c < E ? z[lane + 64 * c] : -INFINITY; m = fmaxf(m, v[c]); }
+        m = wave_max(m);
+        den = 0.0f;
+#pragma unroll
+        for (int c = 0; c < 4; ++c) { v[c] = lane + 64 * c < E ? expf(v[c] - m) : -INFINITY; den += fmaxf(v[c], 0.0f); }
+        den = wave_sum(den);
+    } else {
+#pragma unroll
+        for (int c = 0; c < 4; ++c) v[c] = lane + 64 * c < E ? 1.0f / (1.0f + expf(-z[lane + 64 * c])) : -INFINITY;
+    }
+    if (f.correction) {     // (uniform) what is chosen by is no longer what is weighted with: the scores stay in LDS, v becomes the choice scores
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+            if (lane + 64 * c < E) { const float s = v[c] / den; z[lane + 64 * c] = s; v[c] = s + f.correction[lane + 64 * c]; }
+        __builtin_amdgcn_wave_barrier();
+    }
+    __shared__ int pick_id[kMaxExperts];
+    __shared__ float pick_sc[kMaxExperts];
+    if (f.groups > 1) {
+        // group scores: lane l owns groups l, l + 64, ...: the sum of the group's `group_top` largest scores
+        __shared__ float sc[kMaxExperts];
+        __shared__ unsigned char open_group[kMaxExperts];
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+            if (lane + 64 * c < E) sc[lane + 64 * c] = v[c];
+        __builtin_amdgcn_wave_barrier();
+        const int per = E / f.groups;
+        float gs[4];
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+            const int g = lane + 64 * c;
+            gs[c] = -INFINITY;
+            if (g < f.groups) {
+                float sum = 0.0f;
+                const int nt = min(f.group_top, per);
+                float last = INFINITY;
+                int last_e = -1;
+                for (int k = 0; k < nt; ++k) {                // the largest behind the one before it (equal values: by index)
+                    float best = -INFINITY;
+                    int bi = -1;
+                    for (int e = g * per; e < (g + 1) * per; ++e)
+                        if ((sc[e] < last || (sc[e] == last && e > last_e)) && sc[e] > best) { best = sc[e]; bi = e; }
+                    last = best;
+                    last_e = bi;
+                    sum += best;
+                }
+                gs[c] = sum;
+            }
+            if (g < kMaxExperts) open_group[g] = 0;
+        }
+        __builtin_amdgcn_wave_barrier();
+        for (int k = 0; k < f.keep; ++k) {                    // (taken ones are marked -inf)
+            float bv;
+            int bi;
+            wave_argmax4(gs, lane, bv, bi);
+            if (lane == 0) open_group[bi] = 1;
+            if ((bi & 63) == lane) gs[bi >> 6] = -INFINITY;
+        }
+        __builtin_amdgcn_wave_barrier();
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+            if (lane + 64 * c < E && !open_group[(lane + 64 * c) / per]) v[c] = -INFINITY;
+    }
+    float chosen = 0.0f;
+    for (int s = 0; s < top; ++s) {
+        float bv;
+        int bi;
+        wave_argmax4(v, lane, bv, bi);
+        const float sc1 = f.correction ? z[bi] : bv / den;
+        chosen += sc1;
+        if (lane == 0) { pick_id[s] = bi; pick_sc[s] = sc1; }
+        if ((bi & 63) == lane) v[bi >> 6] = -INFINITY;
+    }
+    const float mul = (f.renorm ? 1.0f / (chosen + 1e-20f) : 1.0f) * f.scale;
+    for (int s = lane; s < top; s += 64) { ids[t * top + s] = pick_id[s]; wts[t * top + s] = pick_sc[s] * mul; }   // (same wave wrote them: in order)
 }
 
 __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, float* wts, float* sgate, float* h, int ldh, const float* wr, const float* wsg,
@@ -74,88 +155,20 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(int* ids, floa
     }
     __syncthreads();
     if (wave != 0) return;
-    // scores and the picks by one wave: lane l holds experts l, l + 64, l + 128, l + 192
-    float v[4];
-    float den = 1.0f;
-    if (f.score == 0) {
-        float m = -INFINITY;
+    pick_experts(z, lane, t, E, top, f, ids, wts);
+}
+
+// the same picks from logits that a product left: z [T][ldz] = [E router outputs | the shared unit's gate (if sgate)], one wave per token
+__global__ __launch_bounds__(64) void moe_pick_kernel(int* ids, float* wts, float* sgate, const float* zg, int ldz, int E, int top, const RouteForm f) {
+    __shared__ float z[kMaxExperts];
+    const int lane = threadIdx.x;
+    const long long t = blockIdx.x;
 #pragma unroll
-        for (int c = 0; c < 4; ++c) { v[c] = lane + 64 * c < E ? z[lane + 64 * c] : -INFINITY; m = fmaxf(m, v[c]); }
-        m = wave_max(m);
-        den = 0.0f;
-#pragma unroll
-        for (int c = 0; c < 4; ++c) { v[c] = lane + 64 * c < E ? expf(v[c] - m) : -INFINITY; den += fmaxf(v[c], 0.0f); }
-        den = wave_sum(den);
-    } else {
-#pragma unroll
-        for (int c = 0; c < 4; ++c) v[c] = lane + 64 * c < E ? 1.0f / (1.0f + expf(-z[lane + 64 * c])) : -INFINITY;
-    }
-    if (f.correction) {     // (uniform) what is chosen by is no longer what is weighted with: the scores stay in LDS, v becomes the choice scores
-#pragma unroll
-        for (int c = 0; c < 4; ++c)
-            if (lane + 64 * c < E) { const float s = v[c] / den; z[lane + 64 * c] = s; v[c] = s + f.correction[lane + 64 * c]; }
-        __builtin_amdgcn_wave_barrier();
-    }
-    __shared__ int pick_id[kMaxExperts];
-    __shared__ float pick_sc[kMaxExperts];
-    if (f.groups > 1) {
-        // group scores: lane l owns groups l, l + 64, ...: the sum of the group's `group_top` largest scores (taken ones are marked -inf)
-        __shared__ float sc[kMaxExperts];
-        __shared__ unsigned char open_group[kMaxExperts];
-#pragma unroll
-        for (int c = 0; c < 4; ++c)
-            if (lane + 64 * c < E) sc[lane + 64 * c] = v[c];
-        __builtin_amdgcn_wave_barrier();
-        const int per = E / f.groups;
-        float gs[4];
-#pragma unroll
-        for (int c = 0; c < 4; ++c) {
-            const int g = lane + 64 * c;
-            gs[c] = -INFINITY;
-            if (g < f.groups) {
-                float sum = 0.0f;
-                int taken[8];
-                const int nt = min(min(f.group_top, per), 8);
-                for (int k = 0; k < nt; ++k) {
-                    float best = -INFINITY;
-                    int bi = -1;
-                    for (int e = g * per; e < (g + 1) * per; ++e) {
-                        bool used = false;
-                        for (int u = 0; u < k; ++u) used = used || taken[u] == e;
-                        if (!used && sc[e] > best) { best = sc[e]; bi = e; }
-                    }
-                    taken[k] = bi;
-                    sum += best;
-                }
-                gs[c] = sum;
-            }
-            if (g < kMaxExperts) open_group[g] = 0;
-        }
-        __builtin_amdgcn_wave_barrier();
-        for (int k = 0; k < f.keep; ++k) {
-            float bv;
-            int bi;
-            wave_argmax4(gs, lane, bv, bi);
-            if (lane == 0) open_group[bi] = 1;
-            if ((bi & 63) == lane) gs[bi >> 6] = -INFINITY;
-        }
-        __builtin_amdgcn_wave_barrier();
-#pragma unroll
-        for (int c = 0; c < 4; ++c)
-            if (lane + 64 * c < E && !open_group[(lane + 64 * c) / per]) v[c] = -INFINITY;
-    }
-    float chosen = 0.0f;
-    for (int s = 0; s < top; ++s) {
-        float bv;
-        int bi;
-        wave_argmax4(v, lane, bv, bi);
-        const float sc1 = f.correction ? z[bi] : bv / den;
-        chosen += sc1;
-        if (lane == 0) { pick_id[s] = bi; pick_sc[s] = sc1; }
-        if ((bi & 63) == lane) v[bi >> 6] = -INFINITY;
-    }
-    const float mul = (f.renorm ? 1.0f / (chosen + 1e-20f) : 1.0f) * f.scale;
-    for (int s = lane; s < top; s += 64) { ids[t * top + s] = pick_id[s]; wts[t * top + s] = pick_sc[s] * mul; }   // (same wave wrote them: in order)
+    for (int c = 0; c < 4; ++c)
+        if (lane + 64 * c < E) z[lane + 64 * c] = zg[t * ldz + lane + 64 * c];
+    if (sgate && lane == 0) sgate[t] = 1.0f / (1.0f + expf(-zg[t * ldz + E]));
+    __syncthreads();
+    pick_experts(z, lane, t, E, top, f, ids, wts);
 }
 
 // Stable counting sort of the pairs by expert, one workgroup of 1024: the pairs are cut into S = 1024 / E' contiguous segments (E' = E rounded up to a
@@ -247,18 +260,34 @@ int ntk_moe_route(int* ids, float* wts, float* sgate, const float* h, int ldh, c
     return ntk_moe_route_ex(ids, wts, sgate, h, ldh, w_router, shared_gate_w, T, n, E, top, &r, stream);
 }
 
+static int route_form(const ntk_route_desc* r, int E, int top, RouteForm* f) {
+    if (r->score != 0 && r->score != 1) return NTK_E_SHAPE;
+    const int groups = r->groups > 1 ? r->groups : 1;
+    if (groups > 1 && (E % groups || r->keep < 1 || r->keep > groups || r->group_top < 1 || r->group_top > 8 || (long long)r->keep * (E / groups) < top)) return NTK_E_SHAPE;
+    *f = RouteForm{r->score, groups, r->keep, r->group_top, r->renorm, r->scale, r->correction, r->add_y, r->ld_add, r->add_w, r->add_eps};
+    return NTK_OK;
+}
+
 int ntk_moe_route_ex(int* ids, float* wts, float* sgate, const float* h, int ldh, const float* w_router, const float* shared_gate_w, int T, int n, int E, int top,
                      const ntk_route_desc* r, void* stream) {
     if (!ids || !wts || !h || !w_router || !r) return NTK_E_NULL;
     if (T < 0 || n <= 0 || E <= 0 || E > kMaxExperts || top <= 0 || top > E || ldh < n) return NTK_E_SHAPE;
-    if (r->score != 0 && r->score != 1) return NTK_E_SHAPE;
     if (r->add_y && (!r->add_w || r->ld_add < n || r->add_y == h)) return NTK_E_SHAPE;
-    const int groups = r->groups > 1 ? r->groups : 1;
-    if (groups > 1 && (E % groups || r->keep < 1 || r->keep > groups || r->group_top < 1 || r->group_top > 8 || (long long)r->keep * (E / groups) < top)) return NTK_E_SHAPE;
-    if (T == 0) return NTK_OK;
     if ((size_t)n * 4 > 128 * 1024) return NTK_E_SHAPE;
-    const RouteForm f{r->score, groups, r->keep, r->group_top, r->renorm, r->scale, r->correction, r->add_y, r->ld_add, r->add_w, r->add_eps};
+    RouteForm f;
+    const int st = route_form(r, E, top, &f);
+    if (st != NTK_OK || T == 0) return st;
     hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(kRouteThreads), (size_t)n * 4, resolve_stream(stream), ids, wts, sgate, (float*)h, ldh, w_router, shared_gate_w, n, E, top, f);
+    return last_launch_status();
+}
+
+int ntk_moe_pick(int* ids, float* wts, float* sgate, const float* z, int ldz, int T, int E, int top, const ntk_route_desc* r, void* stream) {
+    if (!ids || !wts || !z || !r) return NTK_E_NULL;
+    if (T < 0 || E <= 0 || E > kMaxExperts || top <= 0 || top > E || ldz < E + (sgate ? 1 : 0) || r->add_y) return NTK_E_SHAPE;
+    RouteForm f;
+    const int st = route_form(r, E, top, &f);
+    if (st != NTK_OK || T == 0) return st;
+    hipLaunchKernelGGL(moe_pick_kernel, dim3(T), dim3(64), 0, resolve_stream(stream), ids, wts, sgate, z, ldz, E, top, f);
     return last_launch_status();
 }
 

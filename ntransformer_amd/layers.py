@@ -88,6 +88,7 @@ def _bind():
     L.ntk_dense.argtypes = [C.POINTER(DenseDesc), vp]
     L.ntk_embed_sinusoid.argtypes = [vp, vp, i, vp, i, i, i, f, vp, i, vp]
     L.ntk_latent_fold_query_prepare.argtypes = [vp, vp, i, vp, i, i, i, i, i, vp, i, vp, i, vp, f, i, vp]
+    L.ntk_moe_pick.argtypes = [vp, vp, vp, vp, i, i, i, i, C.POINTER(RouteDesc), vp]
     L.ntk_moe_few.argtypes = [C.POINTER(MoeFewDesc), vp]
     L.ntk_moe_sum_ex.argtypes = [vp, vp, vp, vp, i, vp, i, vp, vp, vp, i, i, i, vp]
     L.ntk_dense_linear.argtypes = [vp, i, vp, i, vp, i, i, i, i, i, vp]
@@ -677,6 +678,21 @@ def latent_fold_query_prepare(q: np.ndarray, w_uk: np.ndarray, heads: int, dn: i
     check(L.ntk_latent_fold_query_prepare(out.ptr, qb.ptr, q.shape[1], wb.ptr, dt, T, heads, dn, R, cb.ptr, cache.shape[1], kb.ptr, kv.shape[1], nb.ptr, eps, pos0, None),
           "ntk_latent_fold_query_prepare")
     return out.numpy(np.float32, T * heads * R).reshape(T, heads * R), cb.numpy(np.float32, cache.size).reshape(cache.shape)
+
+
+def moe_pick(z: np.ndarray, E: int, top: int, score: int = 0, groups: int = 1, keep: int = 1, group_top: int = 1, renorm: bool = False, scale: float = 1.0,
+             correction: Optional[np.ndarray] = None):
+    """z [T, E] router outputs, or [T, E + 1] with the shared unit's gate ahead of its sigmoid -> (ids, weights, gates or None)"""
+    L = _bind()
+    T = z.shape[0]
+    zb, ids, wts = _f(z), DeviceBuffer.zeros(T * top * 4), DeviceBuffer.zeros(T * top * 4)
+    sg = DeviceBuffer.zeros(T * 4) if z.shape[1] > E else None
+    r = RouteDesc(score, groups, keep, group_top, int(renorm), scale)
+    if correction is not None:
+        cb = _f(correction)
+        r.correction = cb.ptr
+    check(L.ntk_moe_pick(ids.ptr, wts.ptr, sg.ptr if sg else None, zb.ptr, z.shape[1], T, E, top, C.byref(r), None), "ntk_moe_pick")
+    return ids.numpy(np.int32, T * top).reshape(T, top), wts.numpy(np.float32, T * top).reshape(T, top), (sg.numpy(np.float32, T) if sg else None)
 
 
 def moe_few(h: np.ndarray, ids, wts, up: np.ndarray, down: np.ndarray, shared_up=None, shared_down=None, sgate=None, act: int = ACT_RELU2, dtype: str = "float32") -> np.ndarray:

@@ -265,6 +265,10 @@ def test_router_with_a_correction(E, top, groups, keep):
             want = O.route(wr.astype(F64) @ h[t].astype(F64), corr.astype(F64), top, {"count": groups, "keep": keep} if groups > 1 else None)
             assert list(ids[t]) == [e for e, _ in want], (shift, t)
             assert np.allclose(wts[t], [s for _, s in want], rtol=2e-5, atol=1e-9)
+        z = f32(np.concatenate([h.astype(F64) @ wr.T.astype(F64), g.standard_normal((T, 1))], axis=1))      # the choice alone, behind a product that also formed a gate
+        pids, pw, sg = Lr.moe_pick(z, E, top, groups=groups, keep=keep, correction=corr)
+        assert np.array_equal(pids, ids) and np.allclose(pw, wts, rtol=1e-4, atol=1e-9) and np.allclose(sg, O.sigmoid(z[:, -1].astype(F64)), rtol=1e-6)
+        assert Lr.moe_pick(z[:, :-1], E, top, groups=groups, keep=keep, correction=corr)[2] is None
     ids, wts = Lr.moe_route_ex(np.zeros((2, n), np.float32), wr, top, score=0, groups=groups, keep=keep, group_top=1, correction=np.full(E, -7.0, np.float32))
     assert list(ids[0]) == list(range(top)) and np.allclose(wts, 1.0 / E)
     y, aw = f32(g.standard_normal((T, n)) * 5), f32(1 + 0.3 * g.standard_normal(n))      # what the rows are still owed joins them first
@@ -560,6 +564,7 @@ def _other():
         "half of the choices identity": O.config([A(mlp=M(4, 3, 12, identity=4, groups=(2, 1), shared=8)), L(mlp=M(1, 2, 12, identity=5, groups=(3, 2)))]),
         "many experts": O.config([A(mlp=M(130, 9, 8, identity=14, groups=(12, 5), shared=24)), L(mlp=M(250, 20, 8, identity=5))], vocab=40),
         "six heads (slopes between the powers of two)": O.config([A(6, 2, 20, mlp=D()), A(5, 5, 12, mlp=D()), A(16, 1, 4)], eps=1e-6),
+        "experts wider than one row of activations": O.config([A(mlp=M(3, 2, 18500, identity=1, shared=40)), L(mlp=M(2, 2, 32))], width=8),
         "wider than one register pass": O.config([L(2, 8, 8, 16, mlp=D(16)), A(2, 1, 8, mlp=M(3, 2, 16, identity=1, shared=8))], vocab=20, width=4104),
     }
 
