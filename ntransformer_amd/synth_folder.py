@@ -378,6 +378,8 @@ def write_folder(folder: str, cfg: dict, seed: int = 20260925) -> int:
                 if cfg.get("architecture") in ("Fifotar", "Zalazen", "Gibevik"):     # every norm weight is stored plain; decay rates and biases small
                     around_one = "norm" in name.rsplit(".", 1)[-1]
                 vals = 0.1 * pool[:n] + (1.0 if around_one else 0.0)
+                if name.endswith(".correction"):              # joins scores that average 1 / n: a tenth of that, so that every token does not choose alike
+                    vals = vals / n
                 f.write(_bf16(vals).tobytes())
                 continue
             scale = 1.0 if name == "embed" else 1.0 / math.sqrt(shp[-1])
